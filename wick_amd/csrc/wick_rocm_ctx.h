@@ -73,6 +73,13 @@ inline bool graph_is_stale(const wick_rocm_ctx* ctx, const wick_rocm_graph* g) {
     return false;
 }
 
+// The static scratch array of wick_rocm_matmul_f32_noalloc (context.hip): quants first, scales behind them.
+constexpr size_t kNoallocMaxElems = 4u << 20;  // n * k of one call: 4 Mi quants (4 MiB) + 128 Ki scales (512 KiB)
+constexpr size_t kNoallocScratchBytes = kNoallocMaxElems + kNoallocMaxElems / 32 * sizeof(float);
+// Claims that array for ctx (an error while another context of the same GPU may still be using it) / gives it back.
+int noalloc_claim(wick_rocm_ctx* ctx);
+void noalloc_release(wick_rocm_ctx* ctx);
+
 struct wick_rocm_event {
     hipEvent_t ev = nullptr;
 };

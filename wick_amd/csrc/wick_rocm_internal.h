@@ -12,6 +12,7 @@ namespace wick_rocm {
 
 constexpr int kTypeQ4_0 = 2;  // ggml ids, wick/src/gguf.rs:36-51
 constexpr int kTypeQ8_0 = 8;
+constexpr int kTypeBF16 = 30;  // embedding rows only (token_ops.hip)
 constexpr int kQ4BlockBytes = 18;  // wick/src/quant.rs:13-20
 constexpr int kQ8BlockBytes = 34;  // wick/src/quant.rs:27-34
 constexpr int kMaxGemvBatch = 4;
@@ -159,7 +160,7 @@ hipError_t launch_block_dots_gemv_f32(int type, const uint8_t* d_w, uint32_t m, 
 hipError_t launch_block_dots_mfma(int type, const uint8_t* d_w, uint32_t m, uint32_t k, const int8_t* d_q, uint32_t n,
                                   int32_t* d_out, const Launch& L);
 
-// The non-matmul operations of an LFM2 decode step (lfm2_ops.hip).  d_pos / d_token, when non-null, are read on the
+// The non-matmul operations of an LFM2 decode step (lfm2_ops.hip; embedding rows and the greedy pick: token_ops.hip).  d_pos / d_token, when non-null, are read on the
 // device in place of the by-value pos / token.
 hipError_t launch_embed_row(const uint8_t* d_w, int type, uint32_t m, uint32_t k, uint32_t token, const uint32_t* d_token, float* d_out,
                             const Launch& L);
