@@ -55,6 +55,17 @@ def test_lfm2_step_symbols_are_exported_and_bound():
     assert sorted(lfm2._SIGNATURES) == names
 
 
+def test_model_symbols_are_exported_and_bound():
+    from wick_amd import checkpoint, model
+
+    lib = wick_amd.load_library()
+    for header, prefix, bound in (("wick_rocm_model.h", "wick_rocm_model_", model), ("wick_safetensors.h", "wick_safetensors_", checkpoint)):
+        names = declared_symbols(header, prefix)
+        for name in names:
+            assert hasattr(lib, name), f"{name} declared in {header} but not exported"
+        assert sorted(bound._SIGNATURES) == names
+
+
 def test_static_library_is_built_too():
     """What a Rust build.rs would link (cargo:rustc-link-lib=static=wick_rocm)."""
     assert os.path.exists(os.path.join(ROOT, "wick_amd", "lib", "libwick_rocm.a"))
@@ -113,7 +124,7 @@ def test_documented_build_rs_matches_the_makefile():
     doc = _documented_build()
     srcs, flags, preload_units, preload_flags = _makefile_vars()
     assert [u + ".hip" for u in doc["HIP_UNITS"]] == srcs
-    assert doc["CPP_UNITS"] == ["gguf"]
+    assert doc["CPP_UNITS"] == ["gguf", "safetensors"]
     assert sorted(doc["PRELOAD_UNITS"]) == sorted(preload_units) and doc["PRELOAD_FLAGS"] == preload_flags
     warn = {"-Wall", "-Wno-unused-function"}  # diagnostics only
     assert doc["HIP_FLAGS"] == [f.replace("$(ARCH)", "gfx950") for f in flags if f not in warn]
@@ -137,9 +148,10 @@ def test_archive_of_the_documented_units_links_the_host_mirror(tmp_path):
     out = subprocess.run(["g++", "-O1", "-std=c++17", "-o", exe, os.path.join(ROOT, "wick_amd", "host", "selftest.cpp"), lib,
                           "-L/opt/rocm/lib", "-lamdhip64", "-Wl,-rpath,/opt/rocm/lib", "-lpthread"], capture_output=True, text=True)
     assert out.returncode == 0, out.stderr[-3000:]
-    # and every symbol the three headers declare is defined in that archive
+    # and every symbol the headers declare is defined in that archive
     nm = subprocess.run(["nm", "-g", "--defined-only", lib], capture_output=True, text=True, check=True).stdout
     defined = set(re.findall(r" T (\w+)", nm))
-    for header, prefix in (("wick_rocm.h", "wick_rocm_"), ("wick_rocm_lfm2.h", "wick_rocm_"), ("wick_gguf.h", "wick_gguf_")):
+    for header, prefix in (("wick_rocm.h", "wick_rocm_"), ("wick_rocm_lfm2.h", "wick_rocm_"), ("wick_gguf.h", "wick_gguf_"),
+                           ("wick_rocm_model.h", "wick_rocm_model_"), ("wick_safetensors.h", "wick_safetensors_")):
         for name in declared_symbols(header, prefix):
             assert name in defined, f"{name} ({header}) is not defined by the documented units"

@@ -1,0 +1,378 @@
+// Matrix products of a prompt for bfloat16 weights: out[t][f] = sum_k W[f][k] x[t][k] for n token rows, with what follows the product
+// (bias, activation, gate, the coefficients of a recurrence) in the epilogue.
+//
+// Two bodies share the epilogues, because the 16 x 16 result of v_mfma_f32_16x16x32_bf16 and of v_mfma_f32_16x16x4_f32 sits in the
+// same registers (lane l: column l % 16, rows 4 (l / 16) + r):
+//   gemm_bf16_kernel  activations in bfloat16; 2 x 2 waves of (16 MT) x (16 NT) outputs, K in steps of 64 through two LDS buffers
+//                     (the next step's global loads are in flight during the products of this one); the 16-byte chunks of an LDS
+//                     row are permuted by row % 8, so that the 16 rows a fragment read touches spread over the banks;
+//   gemm_f32_kernel   activations in f32, weights widened exactly: every product and sum in f32.
+// Weights are the M side, so a lane ends with four consecutive features of one token: one vector store.  With TRANS the sides are
+// swapped and a lane holds four consecutive tokens of one feature (a transposed result).
+#include "wick_rocm_dense.h"
+#include "wick_rocm_device.h"
+
+namespace wick_rocm {
+
+namespace {
+
+typedef float v4f __attribute__((ext_vector_type(4)));
+typedef __bf16 bf8 __attribute__((ext_vector_type(8)));
+typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ float bf16_to_f32(uint16_t b) { return __uint_as_float((uint32_t)b << 16); }
+
+__device__ __forceinline__ void store4(float* p, v4f v) { *reinterpret_cast<v4f*>(p) = v; }
+__device__ __forceinline__ void store4(uint16_t* p, v4f v) {
+    bf4 b;
+#pragma unroll
+    for (int i = 0; i < 4; i++) b[i] = (__bf16)v[i];
+    *reinterpret_cast<bf4*>(p) = b;
+}
+
+__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float siluf(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float gelu_tanhf(float z) {
+    // 0.5 (1 + tanh(s)) = 1 / (1 + exp(-2 s))
+    const float s = 0.79788456080286535588f * (z + 0.044715f * z * z * z);
+    return z / (1.0f + expf(-2.0f * s));
+}
+
+// ---- epilogues: (z, first feature, token row of the output, sums[, sums of the second weight]) --------------------------
+struct EpiStore {
+    static constexpr bool kPaired = false, kTrans = false;
+    float* out;
+    uint32_t ldo;
+    const float* add;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f a, v4f) const {
+        if (add) a += *reinterpret_cast<const v4f*>(add + f);
+        store4(out + (size_t)t * ldo + f, a);
+    }
+};
+struct EpiGeluSplit {
+    static constexpr bool kPaired = false, kTrans = false;
+    float* out;
+    uint32_t ldo;
+    const float* bias;
+    uint32_t split;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f a, v4f) const {
+        a += *reinterpret_cast<const v4f*>(bias + f);
+        if (f < split) {
+#pragma unroll
+            for (int i = 0; i < 4; i++) a[i] = gelu_tanhf(a[i]);
+        }
+        store4(out + (size_t)t * ldo + f, a);
+    }
+};
+template <typename AT>
+struct EpiRelu2 {
+    static constexpr bool kPaired = false, kTrans = false;
+    AT* out;
+    uint32_t ldo;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f a, v4f) const {
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const float r = fmaxf(a[i], 0.0f);
+            a[i] = r * r;
+        }
+        store4(out + (size_t)t * ldo + f, a);
+    }
+};
+template <typename AT>
+struct EpiSilu {
+    static constexpr bool kPaired = true, kTrans = false;
+    AT* out;
+    uint32_t ldo;
+    const float* row_scale;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f g, v4f u) const {
+        const float s = row_scale ? row_scale[t] : 1.0f;
+#pragma unroll
+        for (int i = 0; i < 4; i++) g[i] = siluf(g[i]) * u[i] * s;
+        store4(out + (size_t)t * ldo + f, g);
+    }
+};
+template <typename AT>
+struct EpiConvert {
+    static constexpr bool kPaired = false, kTrans = false;
+    AT* out;
+    uint32_t ldo;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f a, v4f) const { store4(out + (size_t)t * ldo + f, a); }
+};
+template <typename AT>
+struct EpiTransposed {  // f: this lane's feature, t: the first of its four tokens
+    static constexpr bool kPaired = false, kTrans = true;
+    AT* out;
+    uint32_t ldo;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f a, v4f) const { store4(out + (size_t)f * ldo + t, a); }
+};
+struct EpiGates {
+    static constexpr bool kPaired = true, kTrans = false;
+    GateArgs g;
+    uint32_t block;
+    __device__ void operator()(uint32_t z, uint32_t f, uint32_t t, v4f r, v4f i) const {
+        const uint32_t ch = z * block + f;
+        const size_t at = (size_t)t * g.channels + ch;
+        r += *reinterpret_cast<const v4f*>(g.r_bias + ch), i += *reinterpret_cast<const v4f*>(g.i_bias + ch);
+        const v4f rate = *reinterpret_cast<const v4f*>(g.rate + ch), u = *reinterpret_cast<const v4f*>(g.u + at);
+        v4f a, b;
+#pragma unroll
+        for (int k = 0; k < 4; k++) {
+            const float log_a = sigmoidf(r[k]) * rate[k];
+            a[k] = expf(log_a);
+            b[k] = sqrtf(-expm1f(2.0f * log_a)) * (sigmoidf(i[k]) * u[k]);
+        }
+        store4(g.a + at, a), store4(g.b + at, b);
+    }
+};
+
+struct GemmArgs {
+    const uint16_t* w;
+    size_t w_stride;     // elements between groups / blocks
+    uint32_t ldw, mp;
+    const void* x;
+    uint32_t ldx, n, k, x_stride_z;
+    Grouping g;
+};
+
+// The workgroup's tile: which weights, which token rows.  false: nothing to do (a grouped launch is sized for the worst case).
+struct TileAt {
+    uint32_t m0, t0, rows, z;   // first feature, first output row, rows present, block
+    const uint16_t* w;
+};
+__device__ __forceinline__ bool tile_at(const GemmArgs& a, uint32_t bm, uint32_t bn, TileAt& o) {
+    uint32_t bid = blockIdx.x;
+    // consecutive workgroups go to the eight XCDs in turn: give every XCD a contiguous run of tiles
+    if (gridDim.x % 8u == 0) bid = (bid & 7u) * (gridDim.x >> 3) + (bid >> 3);
+    const uint32_t mtiles = (a.mp + bm - 1) / bm;
+    const uint32_t nt = bid / mtiles;
+    o.m0 = (bid % mtiles) * bm, o.z = blockIdx.z;
+    o.w = a.w + (size_t)blockIdx.z * a.w_stride;
+    if (a.g.tiles) {
+        if (nt >= *a.g.n_tiles) return false;
+        const GroupTile t = a.g.tiles[nt];
+        o.w = a.w + (size_t)t.group * a.w_stride;
+        o.t0 = t.first, o.rows = t.count;
+    } else {
+        o.t0 = nt * bn;
+        o.rows = a.n - o.t0 < bn ? a.n - o.t0 : bn;
+    }
+    return true;
+}
+__device__ __forceinline__ uint32_t source_row(const GemmArgs& a, const TileAt& o, uint32_t r) {
+    const uint32_t e = o.t0 + (r < o.rows ? r : o.rows - 1u);  // rows past the end repeat the last one and are not stored
+    return a.g.gather ? a.g.gather[e] : e;
+}
+
+template <int MT, int NT, class Epi>
+__device__ __forceinline__ void run_epilogue(const GemmArgs& a, const TileAt& o, const Epi& epi, const v4f (&acc)[MT][NT], uint32_t wm, uint32_t wn,
+                                             uint32_t l16, uint32_t g) {
+    if constexpr (Epi::kTrans) {
+#pragma unroll
+        for (int i = 0; i < MT; i++)
+#pragma unroll
+            for (int j = 0; j < NT; j++) {
+                const uint32_t f = o.m0 + wm + 16 * i + l16, r = wn + 16 * j + 4 * g;
+                if (f < a.mp && r < o.rows) epi(o.z, f, o.t0 + r, acc[i][j], acc[i][j]);  // tokens past the end land in the row's padding
+            }
+    } else {
+#pragma unroll
+        for (int j = 0; j < NT; j++) {
+            const uint32_t r = wn + 16 * j + l16;
+            if (r >= o.rows) continue;
+            if constexpr (Epi::kPaired) {
+#pragma unroll
+                for (int i = 0; i < MT; i += 2) {
+                    const uint32_t row = o.m0 + wm + 16 * i;  // a multiple of 32
+                    if (row < a.mp) epi(o.z, (row >> 1) + 4 * g, o.t0 + r, acc[i][j], acc[i + 1][j]);
+                }
+            } else {
+#pragma unroll
+                for (int i = 0; i < MT; i++) {
+                    const uint32_t f = o.m0 + wm + 16 * i + 4 * g;
+                    if (f < a.mp) epi(o.z, f, o.t0 + r, acc[i][j], acc[i][j]);
+                }
+            }
+        }
+    }
+}
+
+template <int MT, int NT, class Epi>
+__global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
+    constexpr uint32_t BM = 32 * MT, BN = 32 * NT, BK = 64;
+    constexpr int LA = BM * 8 / 256, LB = BN * 8 / 256;  // 16-byte chunks per thread and step
+    __shared__ __align__(16) uint16_t sa[2][BM * BK], sb[2][BN * BK];
+    TileAt o;
+    if (!tile_at(a, BM, BN, o)) return;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, g = lane >> 4;
+    const uint32_t wm = (wave & 1u) * (16 * MT), wn = (wave >> 1) * (16 * NT);
+    const uint16_t* x = static_cast<const uint16_t*>(a.x) + (size_t)o.z * a.x_stride_z;
+    const uint16_t *pa[LA], *pb[LB];
+    uint32_t da[LA], db[LB];
+#pragma unroll
+    for (int i = 0; i < LA; i++) {
+        const uint32_t c = tid + 256 * i, row = c >> 3, ch = c & 7u, m = o.m0 + row < a.mp ? o.m0 + row : a.mp - 1u;
+        pa[i] = o.w + (size_t)m * a.ldw + ch * 8;
+        da[i] = row * BK + ((ch ^ (row & 7u)) << 3);
+    }
+#pragma unroll
+    for (int i = 0; i < LB; i++) {
+        const uint32_t c = tid + 256 * i, row = c >> 3, ch = c & 7u;
+        pb[i] = x + (size_t)source_row(a, o, row) * a.ldx + ch * 8;
+        db[i] = row * BK + ((ch ^ (row & 7u)) << 3);
+    }
+    u4 ra[LA], rb[LB];
+#pragma unroll
+    for (int i = 0; i < LA; i++) ra[i] = *reinterpret_cast<const u4*>(pa[i]);
+#pragma unroll
+    for (int i = 0; i < LB; i++) rb[i] = *reinterpret_cast<const u4*>(pb[i]);
+    v4f acc[MT][NT];
+#pragma unroll
+    for (int i = 0; i < MT; i++)
+#pragma unroll
+        for (int j = 0; j < NT; j++) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < LA; i++) *reinterpret_cast<u4*>(&sa[0][da[i]]) = ra[i];
+#pragma unroll
+    for (int i = 0; i < LB; i++) *reinterpret_cast<u4*>(&sb[0][db[i]]) = rb[i];
+    __syncthreads();
+    int cur = 0;
+    for (uint32_t k0 = 0; k0 < a.k; k0 += BK, cur ^= 1) {
+        const bool more = k0 + BK < a.k;
+        if (more) {
+#pragma unroll
+            for (int i = 0; i < LA; i++) ra[i] = *reinterpret_cast<const u4*>(pa[i] + k0 + BK);
+#pragma unroll
+            for (int i = 0; i < LB; i++) rb[i] = *reinterpret_cast<const u4*>(pb[i] + k0 + BK);
+        }
+#pragma unroll
+        for (int s = 0; s < 2; s++) {
+            bf8 fa[MT], fb[NT];
+            const uint32_t ch = (((4 * s + g) ^ (l16 & 7u)) << 3);
+#pragma unroll
+            for (int i = 0; i < MT; i++) fa[i] = *reinterpret_cast<const bf8*>(&sa[cur][(wm + 16 * i + l16) * BK + ch]);
+#pragma unroll
+            for (int j = 0; j < NT; j++) fb[j] = *reinterpret_cast<const bf8*>(&sb[cur][(wn + 16 * j + l16) * BK + ch]);
+#pragma unroll
+            for (int i = 0; i < MT; i++)
+#pragma unroll
+                for (int j = 0; j < NT; j++)
+                    acc[i][j] = Epi::kTrans ? __builtin_amdgcn_mfma_f32_16x16x32_bf16(fb[j], fa[i], acc[i][j], 0, 0, 0)
+                                            : __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        }
+        if (more) {
+#pragma unroll
+            for (int i = 0; i < LA; i++) *reinterpret_cast<u4*>(&sa[cur ^ 1][da[i]]) = ra[i];
+#pragma unroll
+            for (int i = 0; i < LB; i++) *reinterpret_cast<u4*>(&sb[cur ^ 1][db[i]]) = rb[i];
+        }
+        __syncthreads();
+    }
+    run_epilogue<MT, NT>(a, o, epi, acc, wm, wn, l16, g);
+}
+
+template <class Epi>
+__global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs a, Epi epi) {
+    constexpr int MT = 2, NT = 2;
+    constexpr uint32_t BM = 64, BN = 64, BK = 32, LD = BK + 4;
+    __shared__ __align__(16) float sa[BM * LD], sb[BN * LD];
+    TileAt o;
+    if (!tile_at(a, BM, BN, o)) return;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, g = lane >> 4;
+    const uint32_t wm = (wave & 1u) * 32u, wn = (wave >> 1) * 32u;
+    const float* x = static_cast<const float*>(a.x) + (size_t)o.z * a.x_stride_z;
+    const uint32_t arow = tid >> 2, ach = (tid & 3u) * 8u;
+    const uint16_t* pa = o.w + (size_t)(o.m0 + arow < a.mp ? o.m0 + arow : a.mp - 1u) * a.ldw + ach;
+    const float* pb = x + (size_t)source_row(a, o, arow) * a.ldx + ach;
+    v4f acc[MT][NT];
+#pragma unroll
+    for (int i = 0; i < MT; i++)
+#pragma unroll
+        for (int j = 0; j < NT; j++) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
+    for (uint32_t k0 = 0; k0 < a.k; k0 += BK) {
+        const uint4 wv = *reinterpret_cast<const uint4*>(pa + k0);
+        const v4f b0 = *reinterpret_cast<const v4f*>(pb + k0), b1 = *reinterpret_cast<const v4f*>(pb + k0 + 4);
+        __syncthreads();  // the previous step's reads are done
+        float* da = &sa[arow * LD + ach];
+        const uint32_t wq[4] = {wv.x, wv.y, wv.z, wv.w};
+#pragma unroll
+        for (int i = 0; i < 4; i++) da[2 * i] = __uint_as_float(wq[i] << 16), da[2 * i + 1] = __uint_as_float(wq[i] & 0xffff0000u);
+        *reinterpret_cast<v4f*>(&sb[arow * LD + ach]) = b0, *reinterpret_cast<v4f*>(&sb[arow * LD + ach + 4]) = b1;
+        __syncthreads();
+#pragma unroll
+        for (uint32_t kk = 0; kk < BK; kk += 4) {
+            float fa[MT], fb[NT];
+#pragma unroll
+            for (int i = 0; i < MT; i++) fa[i] = sa[(wm + 16 * i + l16) * LD + kk + g];
+#pragma unroll
+            for (int j = 0; j < NT; j++) fb[j] = sb[(wn + 16 * j + l16) * LD + kk + g];
+#pragma unroll
+            for (int i = 0; i < MT; i++)
+#pragma unroll
+                for (int j = 0; j < NT; j++)
+                    acc[i][j] = Epi::kTrans ? __builtin_amdgcn_mfma_f32_16x16x4f32(fb[j], fa[i], acc[i][j], 0, 0, 0)
+                                            : __builtin_amdgcn_mfma_f32_16x16x4f32(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        }
+    }
+    run_epilogue<MT, NT>(a, o, epi, acc, wm, wn, l16, g);
+}
+
+// Host-side shape checks every launch goes through: K in whole steps, vector-aligned rows.
+bool shapes_fit(const DenseWeight& w, const GemmIn& in, uint32_t k) {
+    return w.d && in.x && w.mp % kDensePad == 0 && k % kDensePad == 0 && w.kp % 8u == 0 && k <= w.kp && in.ldx % 8u == 0 &&
+           (reinterpret_cast<uintptr_t>(w.d) | reinterpret_cast<uintptr_t>(in.x)) % 16u == 0;
+}
+
+template <class Epi>
+hipError_t run_gemm(const DenseWeight& w, const GemmIn& in, const Epi& epi, const Launch& L, const Grouping& g = Grouping(), uint32_t z = 1,
+                    uint32_t x_stride_z = 0) {
+    if (in.n == 0) return hipSuccess;
+    if (!shapes_fit(w, in, w.kp) || (g.tiles && (z != 1 || !g.n_tiles || g.max_tiles == 0))) return hipErrorInvalidValue;
+    const GemmArgs a{w.d, w.stride, w.kp, w.mp, in.x, in.ldx, in.n, w.kp, x_stride_z, g};
+    auto grid = [&](uint32_t bm, uint32_t bn) {
+        const uint32_t mt = (w.mp + bm - 1) / bm, nt = g.tiles ? g.max_tiles : (in.n + bn - 1) / bn;
+        return dim3(mt * nt, 1, z);
+    };
+    if (in.f32) return launch_kernel(L, kFamGemm, gemm_f32_kernel<Epi>, grid(64, 64), dim3(256), a, epi);
+    if (g.tiles) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, Epi>, grid(128, kGroupTileRows), dim3(256), a, epi);
+    const dim3 big = grid(128, 128);
+    if (big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, Epi>, big, dim3(256), a, epi);
+    return launch_kernel(L, kFamGemm, gemm_bf16_kernel<2, 2, Epi>, grid(64, 64), dim3(256), a, epi);
+}
+
+}  // namespace
+
+hipError_t launch_gemm_store(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* add, const Launch& L, const Grouping& g) {
+    if (ldo < w.mp || ldo % 4u) return hipErrorInvalidValue;
+    return run_gemm(w, in, EpiStore{out, ldo, add}, L, g);
+}
+
+hipError_t launch_gemm_gelu_split(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* bias, uint32_t split, const Launch& L) {
+    if (ldo < w.mp || ldo % 4u || split % 4u) return hipErrorInvalidValue;
+    return run_gemm(w, in, EpiGeluSplit{out, ldo, bias, split}, L);
+}
+
+hipError_t launch_gemm_relu2(const DenseWeight& w, const GemmIn& in, void* out, uint32_t ldo, const Launch& L) {
+    if (ldo < w.mp || ldo % 8u) return hipErrorInvalidValue;
+    return in.f32 ? run_gemm(w, in, EpiRelu2<float>{static_cast<float*>(out), ldo}, L)
+                  : run_gemm(w, in, EpiRelu2<uint16_t>{static_cast<uint16_t*>(out), ldo}, L);
+}
+
+hipError_t launch_gemm_silu(const DenseWeight& w, const GemmIn& in, void* out, uint32_t ldo, const float* row_scale, const Launch& L, const Grouping& g) {
+    if (ldo < w.mp / 2u || ldo % 8u) return hipErrorInvalidValue;
+    return in.f32 ? run_gemm(w, in, EpiSilu<float>{static_cast<float*>(out), ldo, row_scale}, L, g)
+                  : run_gemm(w, in, EpiSilu<uint16_t>{static_cast<uint16_t*>(out), ldo, row_scale}, L, g);
+}
+
+hipError_t launch_gemm_convert(const DenseWeight& w, const GemmIn& in, void* out, uint32_t ldo, bool transposed, const Launch& L) {
+    if (in.f32 || ldo % 8u || ldo < (transposed ? pad_to(in.n, 4) : w.mp)) return hipErrorInvalidValue;
+    uint16_t* o = static_cast<uint16_t*>(out);
+    return transposed ? run_gemm(w, in, EpiTransposed<uint16_t>{o, ldo}, L) : run_gemm(w, in, EpiConvert<uint16_t>{o, ldo}, L);
+}
+
+hipError_t launch_gemm_gates(const DenseWeight& w, const GemmIn& in, uint32_t blocks, uint32_t x_block_stride, const GateArgs& g, const Launch& L) {
+    if (blocks == 0 || w.mp / 2u * blocks != g.channels || x_block_stride % 8u || x_block_stride < w.kp) return hipErrorInvalidValue;
+    return run_gemm(w, in, EpiGates{g, w.mp / 2u}, L, Grouping(), blocks, x_block_stride);
+}
+
+}  // namespace wick_rocm

@@ -1,0 +1,364 @@
+// Matrix-vector products of one token over bfloat16 weights with f32 activations: every product and sum in f32, the weights widened
+// exactly.  What comes in front of the product runs in every workgroup's prologue (a few KB out of the L2 each, instead of a launch
+// of its own): the residual update with the norm behind the previous sublayer, the norm in front of this one, the input convolution,
+// the loop's entry.  The first workgroup also keeps what later launches need: the new residual row and the convolution's newest input.
+//
+// A wave takes R output rows; its first weight loads are issued before the prologue, whose latency they share.
+#include "wick_rocm_dense.h"
+#include "wick_rocm_device.h"
+
+namespace wick_rocm {
+
+namespace {
+
+constexpr uint32_t kThreads = 256;
+constexpr uint32_t kGemvMaxK = 15360;  // floats of LDS for the vector
+
+__device__ __forceinline__ float gelu_tanhf(float z) {
+    const float s = 0.79788456080286535588f * (z + 0.044715f * z * z * z);
+    return z / (1.0f + expf(-2.0f * s));
+}
+__device__ __forceinline__ float siluf(float z) { return z / (1.0f + expf(-z)); }
+
+__device__ __forceinline__ float dot8(uint4 w, float4 a, float4 b, float acc) {
+    acc = fmaf(__uint_as_float(w.x << 16), a.x, acc);
+    acc = fmaf(__uint_as_float(w.x & 0xffff0000u), a.y, acc);
+    acc = fmaf(__uint_as_float(w.y << 16), a.z, acc);
+    acc = fmaf(__uint_as_float(w.y & 0xffff0000u), a.w, acc);
+    acc = fmaf(__uint_as_float(w.z << 16), b.x, acc);
+    acc = fmaf(__uint_as_float(w.z & 0xffff0000u), b.y, acc);
+    acc = fmaf(__uint_as_float(w.w << 16), b.z, acc);
+    return fmaf(__uint_as_float(w.w & 0xffff0000u), b.w, acc);
+}
+
+__device__ __forceinline__ float block_sum_f32(float v, float* slots) {
+    v = wave_sum_f32(v);
+    __syncthreads();  // slots may still be read from an earlier call
+    if ((threadIdx.x & 63u) == 0) slots[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (slots[0] + slots[1]) + (slots[2] + slots[3]);
+}
+
+enum { kProVec = 0, kProRow = 1, kProRowConv = 2, kProLoop = 3 };
+
+// Fills vec[0 .. k): the vector itself, the row stage's h, or [x | 0 | x0 | 0].  All threads call it; it ends with a barrier.
+// NE: elements of a row per thread (dim <= 256 NE).
+template <int PRO, int NE>
+__device__ __forceinline__ void fill_vector(const GemvIn& in, uint32_t k, float* vec, float* slots) {
+    const uint32_t tid = threadIdx.x;
+    if constexpr (PRO == kProVec) {
+        for (uint32_t e = tid; e < k; e += kThreads) vec[e] = e < in.vec_len ? in.vec[e] : 0.0f;
+        __syncthreads();
+        return;
+    } else {
+        const RowStage& s = in.row;
+        const bool first = blockIdx.x == 0;
+        float x[NE], y[NE];
+#pragma unroll
+        for (int i = 0; i < NE; i++) {
+            const uint32_t e = tid + kThreads * i;
+            x[i] = e < s.dim ? s.x[e] : 0.0f;
+            y[i] = s.y && e < s.dim ? s.y[e] : 0.0f;
+        }
+        // the inputs of the earlier taps and the convolution's weights are requested before the reductions wait
+        constexpr int TP = PRO == kProRowConv ? 4 : 1;  // taps kept in registers; more are read when they are used
+        float past[TP][NE], cw[TP][NE];
+        uint32_t pos = 0;
+        if constexpr (PRO == kProRowConv) {
+            pos = *in.d_pos;
+#pragma unroll
+            for (int j = 0; j < TP; j++)
+#pragma unroll
+                for (int i = 0; i < NE; i++) {
+                    const uint32_t e = tid + kThreads * i;
+                    const bool on = j < (int)s.taps && e < s.dim;
+                    cw[j][i] = on ? s.conv[(size_t)j * s.dim + e] : 0.0f;
+                    const uint32_t back = s.taps - 1u - (uint32_t)j;  // this tap's distance
+                    past[j][i] = on && back > 0 && pos >= back ? s.ring[(size_t)((pos - back) % s.taps) * s.dim + e] : 0.0f;
+                }
+        }
+        if (s.y) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NE; i++) ss += y[i] * y[i];
+            const float sy = s.g_post / sqrtf(block_sum_f32(ss, slots) / (float)s.dim + s.eps);
+#pragma unroll
+            for (int i = 0; i < NE; i++) x[i] += y[i] * sy;
+        }
+        if (s.x_out && first) {
+#pragma unroll
+            for (int i = 0; i < NE; i++) {
+                const uint32_t e = tid + kThreads * i;
+                if (e < s.dim) s.x_out[e] = x[i];
+            }
+        }
+        if constexpr (PRO == kProLoop) {
+#pragma unroll
+            for (int i = 0; i < NE; i++) {
+                const uint32_t e = tid + kThreads * i;
+                if (e < s.dim) vec[e] = x[i], vec[in.x0_at + e] = in.x0[e];
+            }
+            for (uint32_t e = s.dim + tid; e < in.x0_at; e += kThreads) vec[e] = 0.0f;
+            for (uint32_t e = in.x0_at + s.dim + tid; e < k; e += kThreads) vec[e] = 0.0f;
+        } else {
+            float ss = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NE; i++) ss += x[i] * x[i];
+            const float sx = s.g_pre / sqrtf(block_sum_f32(ss, slots) / (float)s.dim + s.eps);
+#pragma unroll
+            for (int i = 0; i < NE; i++) {
+                const uint32_t e = tid + kThreads * i;
+                if (e >= s.dim) continue;
+                float h = x[i] * sx;
+                if constexpr (PRO == kProRowConv) {
+                    if (first) s.ring[(size_t)(pos % s.taps) * s.dim + e] = h;
+                    float c = 0.0f;
+#pragma unroll
+                    for (int j = 0; j < TP; j++)
+                        if (j < (int)s.taps) c += cw[j][i] * (j + 1 == (int)s.taps ? h : past[j][i]);
+                    for (uint32_t j = TP; j < s.taps; j++) {
+                        const uint32_t back = s.taps - 1u - j;
+                        const float v = back == 0 ? h : pos >= back ? s.ring[(size_t)((pos - back) % s.taps) * s.dim + e] : 0.0f;
+                        c += s.conv[(size_t)j * s.dim + e] * v;
+                    }
+                    h += c;
+                }
+                vec[e] = h;
+            }
+            for (uint32_t e = s.dim + tid; e < k; e += kThreads) vec[e] = 0.0f;
+        }
+        __syncthreads();
+    }
+}
+
+// Weight pieces of N rows that a wave requests before its workgroup's prologue: the first 1024 columns.
+template <int N>
+struct Ahead {
+    uint4 w[N][2];
+    __device__ __forceinline__ void load(const uint16_t* const (&rows)[N], uint32_t k) {
+        const uint32_t at = 8u * (threadIdx.x & 63u);
+#pragma unroll
+        for (int c = 0; c < 2; c++)
+#pragma unroll
+            for (int r = 0; r < N; r++) w[r][c] = at + 512u * c < k ? *reinterpret_cast<const uint4*>(rows[r] + at + 512u * c) : uint4{0, 0, 0, 0};
+    }
+};
+
+// acc[r] += this lane's share of rows[r] . vec over [0, k); AHEAD: the first 1024 columns are in `a` already.
+template <int N, bool AHEAD>
+__device__ __forceinline__ void dot_rows(const uint16_t* const (&rows)[N], const Ahead<N>* a, const float* vec, uint32_t k, float (&acc)[N]) {
+    uint32_t at = 8u * (threadIdx.x & 63u);
+    if constexpr (AHEAD) {
+#pragma unroll
+        for (int c = 0; c < 2; c++) {
+            if (at < k) {
+                const float4 v0 = *reinterpret_cast<const float4*>(vec + at), v1 = *reinterpret_cast<const float4*>(vec + at + 4);
+#pragma unroll
+                for (int r = 0; r < N; r++) acc[r] = dot8(a->w[r][c], v0, v1, acc[r]);
+            }
+            at += 512u;
+        }
+    }
+#pragma unroll 2
+    for (; at < k; at += 512u) {
+        uint4 w[N];
+#pragma unroll
+        for (int r = 0; r < N; r++) w[r] = *reinterpret_cast<const uint4*>(rows[r] + at);
+        const float4 v0 = *reinterpret_cast<const float4*>(vec + at), v1 = *reinterpret_cast<const float4*>(vec + at + 4);
+#pragma unroll
+        for (int r = 0; r < N; r++) acc[r] = dot8(w[r], v0, v1, acc[r]);
+    }
+}
+
+struct DenseArgs {
+    const uint16_t* w;
+    uint32_t ldw, m, k;
+    GemvIn in;
+    float* out;
+    const float* bias;
+    int act;
+    uint32_t split;
+};
+
+template <int PRO, int NE, int R>
+__global__ __launch_bounds__(256) void gemv_dense_kernel(DenseArgs a) {
+    extern __shared__ __align__(16) float vec[];
+    __shared__ float slots[4];
+    const uint32_t lane = threadIdx.x & 63u, row0 = (blockIdx.x * 4u + (threadIdx.x >> 6)) * R;
+    const uint16_t* rows[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) rows[r] = a.w + (size_t)(row0 + r < a.m ? row0 + r : a.m - 1u) * a.ldw;
+    Ahead<R> ahead;
+    ahead.load(rows, a.k);
+    fill_vector<PRO, NE>(a.in, a.k, vec, slots);
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = 0.0f;
+    dot_rows<R, true>(rows, &ahead, vec, a.k, acc);
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        float v = wave_sum_f32(acc[r]);
+        const uint32_t row = row0 + r;
+        if (lane != 0 || row >= a.m) continue;
+        if (a.bias) v += a.bias[row];
+        if (a.act == kActGeluSplit && row < a.split) v = gelu_tanhf(v);
+        if (a.act == kActRelu2) v = fmaxf(v, 0.0f), v = v * v;
+        a.out[row] = v;
+    }
+}
+
+struct RoutedArgs {
+    RoutedMlp m;
+    GemvIn in;
+    const uint32_t* d_token;
+    const float* act_in;
+    float* out;
+    uint32_t k, rows;
+};
+
+__device__ __forceinline__ uint32_t routed_expert(const RoutedArgs& a, uint32_t s) { return (uint32_t)a.m.table[(size_t)*a.d_token * a.m.top + s]; }
+
+template <int NE, int R>
+__global__ __launch_bounds__(256) void gemv_routed_up_kernel(RoutedArgs a) {
+    extern __shared__ __align__(16) float vec[];
+    __shared__ float slots[4];
+    const RoutedMlp& m = a.m;
+    const uint32_t lane = threadIdx.x & 63u, f0 = (blockIdx.x * 4u + (threadIdx.x >> 6)) * R;
+    const uint32_t ff = m.gate_up.mp / 2u, routed = m.top * ff, shared = m.shared_gate_up.d ? m.shared_gate_up.mp / 2u : 0u, total = routed + shared;
+    // this wave's R features lie inside one expert: R divides 16, every expert's width is a multiple of 64
+    const uint16_t* base = m.gate_up.d;
+    uint32_t f = 0, ldw = a.k;
+    if (f0 < routed) {
+        base = m.gate_up.d + (size_t)routed_expert(a, f0 / ff) * m.gate_up.stride, f = f0 % ff;
+    } else if (f0 < total) {
+        base = m.shared_gate_up.d, f = f0 - routed;
+    } else if (f0 == total && shared) {
+        base = m.shared_sg, ldw = 0;  // one row, the same for every r
+    }
+    const uint16_t* rows[2 * R];
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const uint32_t fr = f + r;
+        rows[2 * r] = base + (size_t)((fr >> 4) * 32u + (fr & 15u)) * ldw;
+        rows[2 * r + 1] = base + (size_t)((fr >> 4) * 32u + 16u + (fr & 15u)) * ldw;
+    }
+    Ahead<2 * R> ahead;
+    ahead.load(rows, a.k);
+    fill_vector<kProRow, NE>(a.in, a.k, vec, slots);
+    if (f0 > total || (f0 == total && !shared)) return;
+    float acc[2 * R];
+#pragma unroll
+    for (int r = 0; r < 2 * R; r++) acc[r] = 0.0f;
+    dot_rows<2 * R, true>(rows, &ahead, vec, a.k, acc);
+    if (f0 == total) {
+        const float g = wave_sum_f32(acc[0]);
+        if (lane == 0) a.out[total] = 1.0f / (1.0f + expf(-g));
+        return;
+    }
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const float g = wave_sum_f32(acc[2 * r]), u = wave_sum_f32(acc[2 * r + 1]);
+        if (lane == 0) a.out[f0 + r] = siluf(g) * u;
+    }
+}
+
+template <int R>
+__global__ __launch_bounds__(256) void gemv_routed_down_kernel(RoutedArgs a) {
+    extern __shared__ __align__(16) float vec[];
+    const RoutedMlp& m = a.m;
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, row0 = (blockIdx.x * 4u + (tid >> 6)) * R;
+    const uint32_t ff = m.down.kp, routed = m.top * ff, shared = m.shared_down.d ? m.shared_down.kp : 0u, total = routed + shared;
+    const float share = 1.0f / (float)m.top, gate = shared ? a.act_in[total] : 0.0f;
+    for (uint32_t e = tid; e < total; e += kThreads) vec[e] = a.act_in[e] * (e < routed ? share : gate);
+    __syncthreads();
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = 0.0f;
+    const uint16_t* rows[R];
+    for (uint32_t s = 0; s < m.top; s++) {
+        const uint16_t* base = m.down.d + (size_t)routed_expert(a, s) * m.down.stride;
+#pragma unroll
+        for (int r = 0; r < R; r++) rows[r] = base + (size_t)(row0 + r < a.rows ? row0 + r : a.rows - 1u) * ff;
+        dot_rows<R, false>(rows, nullptr, vec + s * ff, ff, acc);
+    }
+    if (shared) {
+#pragma unroll
+        for (int r = 0; r < R; r++) rows[r] = m.shared_down.d + (size_t)(row0 + r < a.rows ? row0 + r : a.rows - 1u) * shared;
+        dot_rows<R, false>(rows, nullptr, vec + routed, shared, acc);
+    }
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const float v = wave_sum_f32(acc[r]);
+        if (lane == 0 && row0 + r < a.rows) a.out[row0 + r] = v;
+    }
+}
+
+template <int PRO, int NE>
+hipError_t run_dense(const DenseArgs& a, const Launch& L) {
+    const uint32_t lds = a.k * 4u;
+    if (a.m <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NE, 1>, dim3((a.m + 3u) / 4u), dim3(kThreads), lds, a);
+    if (a.m <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NE, 2>, dim3((a.m + 7u) / 8u), dim3(kThreads), lds, a);
+    return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NE, 4>, dim3((a.m + 15u) / 16u), dim3(kThreads), lds, a);
+}
+
+template <int PRO>
+hipError_t run_dense_ne(const DenseArgs& a, const Launch& L) {
+    const uint32_t dim = a.in.row.dim;
+    if (dim <= 1024u) return run_dense<PRO, 4>(a, L);
+    if (dim <= 2048u) return run_dense<PRO, 8>(a, L);
+    if (dim <= 4096u) return run_dense<PRO, 16>(a, L);
+    if (dim <= 8192u) return run_dense<PRO, 32>(a, L);
+    return hipErrorInvalidValue;
+}
+
+bool row_ok(const RowStage& s, uint32_t k) {
+    return s.x && s.dim > 0 && s.dim <= k && s.x_out != s.x && (!s.conv || (s.ring && s.taps > 0)) && !s.experts;
+}
+
+}  // namespace
+
+hipError_t launch_gemv_dense(const DenseWeight& w, uint32_t m, const GemvIn& in, float* out, const float* bias, int act, uint32_t split, const Launch& L) {
+    DenseArgs a{w.d, w.kp, m, in.k ? in.k : w.kp, in, out, bias, act, split};
+    if (!w.d || !out || m == 0 || m > w.mp || a.k > w.kp || a.k % 8u || a.k > kGemvMaxK || w.kp % 8u) return hipErrorInvalidValue;
+    if (in.vec) {
+        if (a.in.vec_len == 0) a.in.vec_len = a.k;
+        return run_dense<kProVec, 1>(a, L);
+    }
+    if (!row_ok(in.row, a.k) || (in.row.conv && !in.d_pos)) return hipErrorInvalidValue;
+    if (in.x0) {
+        if (in.x0_at < in.row.dim || in.x0_at + in.row.dim > a.k) return hipErrorInvalidValue;
+        return run_dense_ne<kProLoop>(a, L);
+    }
+    return in.row.conv ? run_dense_ne<kProRowConv>(a, L) : run_dense_ne<kProRow>(a, L);
+}
+
+uint32_t routed_act_floats(const RoutedMlp& m) { return m.top * (m.gate_up.mp / 2u) + (m.shared_gate_up.d ? m.shared_gate_up.mp / 2u : 0u) + 4u; }
+
+hipError_t launch_gemv_routed_up(const RoutedMlp& m, const GemvIn& in, const uint32_t* d_token, float* act, const Launch& L) {
+    RoutedArgs a{m, in, d_token, nullptr, act, m.gate_up.kp, 0};
+    const bool shared = m.shared_gate_up.d != nullptr;
+    if (!m.gate_up.d || !m.table || m.top == 0 || !d_token || !row_ok(in.row, a.k) || in.row.conv || a.k > kGemvMaxK ||
+        (shared && (m.shared_gate_up.kp != a.k || !m.shared_sg)))
+        return hipErrorInvalidValue;
+    constexpr uint32_t R = 2;
+    const uint32_t features = routed_act_floats(m) - 4u, waves = features / R + 1u;
+    const dim3 grid((waves + 3u) / 4u);
+    const uint32_t lds = a.k * 4u, dim = in.row.dim;
+    if (dim <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<4, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 2048u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<8, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 4096u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<16, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<32, R>, grid, dim3(kThreads), lds, a);
+    return hipErrorInvalidValue;
+}
+
+hipError_t launch_gemv_routed_down(const RoutedMlp& m, uint32_t rows, const float* act, const uint32_t* d_token, float* out, const Launch& L) {
+    RoutedArgs a{m, GemvIn(), d_token, act, out, 0, rows};
+    const uint32_t total = m.top * m.down.kp + (m.shared_down.d ? m.shared_down.kp : 0u);
+    if (!m.down.d || rows == 0 || rows > m.down.mp || m.down.kp != m.gate_up.mp / 2u || total > kGemvMaxK || !d_token ||
+        (m.shared_down.d && m.shared_down.kp != m.shared_gate_up.mp / 2u))
+        return hipErrorInvalidValue;
+    if (rows <= 2048u) return launch_kernel_lds(L, kFamGemv, gemv_routed_down_kernel<1>, dim3((rows + 3u) / 4u), dim3(kThreads), total * 4u, a);
+    return launch_kernel_lds(L, kFamGemv, gemv_routed_down_kernel<2>, dim3((rows + 7u) / 8u), dim3(kThreads), total * 4u, a);
+}
+
+}  // namespace wick_rocm

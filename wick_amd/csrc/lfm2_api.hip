@@ -10,6 +10,7 @@
 #include <vector>
 
 #include "../../include/wick_gguf.h"
+#include "model.h"
 #include "wick_rocm_ctx.h"
 
 namespace {
@@ -483,40 +484,9 @@ int enqueue_step(wick_rocm_ctx* ctx, wick_rocm_lfm2* m, StepMode mode) {
                                  m->d_history, c.max_seq_len, m->hidden);
 }
 
-int step_graph(wick_rocm_ctx* ctx, wick_rocm_lfm2* m, StepMode mode, wick_rocm_graph** out) {
-    wick_rocm_graph*& g = m->g_step[mode];
-    if (g && graph_is_stale(ctx, g)) {  // the context's scratch moved since the capture (another model, a wider matmul): capture again
-        wick_rocm_graph_destroy(ctx, g);
-        g = nullptr;
-    }
-    if (!g) {
-        if (int rc = wick_rocm_graph_begin(ctx)) return rc;
-        const int rc = enqueue_step(ctx, m, mode);
-        wick_rocm_graph* captured = nullptr;
-        const int rc_end = wick_rocm_graph_end(ctx, &captured);  // always end the capture
-        if (rc) {
-            if (captured) wick_rocm_graph_destroy(ctx, captured);
-            return rc;
-        }
-        if (rc_end) return rc_end;
-        g = captured;
-    }
-    *out = g;
-    return WICK_ROCM_OK;
-}
-
 // One step on the context's stream: a replay of the captured graph, or the same launches enqueued one by one.
 int run_step(wick_rocm_ctx* ctx, wick_rocm_lfm2* m, StepMode mode) {
-    // per-dispatch timing cannot see inside a graph: while it is on, steps are enqueued launch by launch
-    bool timing;
-    {
-        std::lock_guard<std::recursive_mutex> lk(ctx->mu);
-        timing = ctx->timer.enabled;
-    }
-    if (!m->use_graph || timing) return enqueue_step(ctx, m, mode);
-    wick_rocm_graph* g = nullptr;
-    if (int rc = step_graph(ctx, m, mode, &g)) return rc;
-    return wick_rocm_graph_launch(ctx, g);
+    return run_step_graph(ctx, m->g_step[mode], m->use_graph, [&] { return enqueue_step(ctx, m, mode); });
 }
 
 constexpr uint32_t kPromptAsStepsMax = 2;  // prompts this short run as single steps (prefill_locked)

@@ -694,31 +694,6 @@ __device__ __forceinline__ void split_f16(float x, _Float16& hi, _Float16& lo) {
     lo = (_Float16)(x - (float)hi);
 }
 
-// Reductions over the four lane groups of a query (lanes l, l ^ 16, l ^ 32, l ^ 48) with gfx950's row / half swaps: swapping a
-// register with a copy of itself leaves the two partners' values in the pair, so their maximum (or sum) needs no select
-// and no trip through the LDS crossbar.  Every lane ends with the result.
-__device__ __forceinline__ float groups_max(float v) {
-    const uint32_t b = __float_as_uint(v);
-    auto r = __builtin_amdgcn_permlane16_swap(b, b, false, false);
-    v = fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
-    const uint32_t c = __float_as_uint(v);
-    auto q = __builtin_amdgcn_permlane32_swap(c, c, false, false);
-    return fmaxf(__uint_as_float(q[0]), __uint_as_float(q[1]));
-}
-__device__ __forceinline__ float groups_sum(float v) {
-    const uint32_t b = __float_as_uint(v);
-    auto r = __builtin_amdgcn_permlane16_swap(b, b, false, false);
-    v = __uint_as_float(r[0]) + __uint_as_float(r[1]);
-    const uint32_t c = __float_as_uint(v);
-    auto q = __builtin_amdgcn_permlane32_swap(c, c, false, false);
-    return __uint_as_float(q[0]) + __uint_as_float(q[1]);
-}
-
-// exp(x) for x <= 0 (-inf included) on the hardware's exp2 (v_exp_f32, about one ulp): two instructions where the polynomial of
-// ggml_expf takes about thirty, and the softmax of a tile is nine of them per lane.  The weights differ from ggml_expf's in the
-// last bit or two; the streaming softmax of this kernel differs from the reference's two-pass one at that level anyway.
-__device__ __forceinline__ float exp_nonpos_hw(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896340736f); }
-
 // KV = _Float16 (f16 caches): K and V are their own high halves and have no low halves, so the K_lo Q_hi and V_lo P_hi
 // products, their operand reads and the low planes' LDS writes drop out (8 of the 12 MFMAs per wave and tile remain).
 template <int HALVES, typename KV>

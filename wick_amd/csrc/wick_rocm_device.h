@@ -231,6 +231,31 @@ __device__ __forceinline__ float wave_max_f32(float v) {
     return fmaxf(fmaxf(r0, r1), fmaxf(r2, r3));
 }
 
+// Reductions over the four lane groups of a query (lanes l, l ^ 16, l ^ 32, l ^ 48) with gfx950's row / half swaps: swapping a
+// register with a copy of itself leaves the two partners' values in the pair, so their maximum (or sum) needs no select
+// and no trip through the LDS crossbar.  Every lane ends with the result.
+__device__ __forceinline__ float groups_max(float v) {
+    const uint32_t b = __float_as_uint(v);
+    auto r = __builtin_amdgcn_permlane16_swap(b, b, false, false);
+    v = fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
+    const uint32_t c = __float_as_uint(v);
+    auto q = __builtin_amdgcn_permlane32_swap(c, c, false, false);
+    return fmaxf(__uint_as_float(q[0]), __uint_as_float(q[1]));
+}
+__device__ __forceinline__ float groups_sum(float v) {
+    const uint32_t b = __float_as_uint(v);
+    auto r = __builtin_amdgcn_permlane16_swap(b, b, false, false);
+    v = __uint_as_float(r[0]) + __uint_as_float(r[1]);
+    const uint32_t c = __float_as_uint(v);
+    auto q = __builtin_amdgcn_permlane32_swap(c, c, false, false);
+    return __uint_as_float(q[0]) + __uint_as_float(q[1]);
+}
+
+// exp(x) for x <= 0 (-inf included) on the hardware's exp2 (v_exp_f32, about one ulp): two instructions where the polynomial of
+// ggml_expf takes about thirty, and the softmax of a tile is nine of them per lane.  The weights differ from ggml_expf's in the
+// last bit or two; the streaming softmax of this kernel differs from the reference's two-pass one at that level anyway.
+__device__ __forceinline__ float exp_nonpos_hw(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896340736f); }
+
 // The greedy pick's ordering (cpu_argmax, wick/src/sampler.rs:7-19) as one unsigned key: NaN counts as -inf, values order
 // by f32::total_cmp, and of equal values the larger index wins; 0 is below every real key.
 __device__ __forceinline__ unsigned long long argmax_key(float f, uint32_t index) {

@@ -52,9 +52,10 @@ struct Launch {
     bool gemm_mfma16 = false;            // plain wide GEMM launches: the 16x16x32 block loop instead of the 32x32x32 one
 };
 
+// `lds`: dynamic LDS bytes of the launch.
 template <typename... KArgs, typename... Args>
-inline hipError_t launch_kernel(const Launch& L, int family, void (*kernel)(KArgs...), dim3 grid, dim3 block,
-                                Args... args) {
+inline hipError_t launch_kernel_lds(const Launch& L, int family, void (*kernel)(KArgs...), dim3 grid, dim3 block, uint32_t lds,
+                                    Args... args) {
     if (L.timer && L.timer->enabled) {
         KernelTimer::Rec r{};
         if (!L.timer->spares.empty()) {
@@ -67,12 +68,16 @@ inline hipError_t launch_kernel(const Launch& L, int family, void (*kernel)(KArg
             if (e != hipSuccess) return e;
         }
         r.family = family;
-        hipExtLaunchKernelGGL(kernel, grid, block, 0, L.stream, r.start, r.stop, 0, args...);
+        hipExtLaunchKernelGGL(kernel, grid, block, lds, L.stream, r.start, r.stop, 0, args...);
         L.timer->recs.push_back(r);
     } else {
-        hipLaunchKernelGGL(kernel, grid, block, 0, L.stream, args...);
+        hipLaunchKernelGGL(kernel, grid, block, lds, L.stream, args...);
     }
     return hipGetLastError();
+}
+template <typename... KArgs, typename... Args>
+inline hipError_t launch_kernel(const Launch& L, int family, void (*kernel)(KArgs...), dim3 grid, dim3 block, Args... args) {
+    return launch_kernel_lds(L, family, kernel, grid, block, 0u, args...);
 }
 
 // Launchers.  All only enqueue on L.stream; callers have validated shapes.
