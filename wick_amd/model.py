@@ -158,7 +158,7 @@ def generate(model: RocmModel, prompt: Sequence[int], max_new: int, stop: Sequen
     _, logits = model.prefill_chunked(prompt, start_pos, ubatch)
     pos = start_pos + len(prompt)
     out = [greedy_pick(logits) if sample is None else int(sample(logits))]
-    stops = set(int(s) for s in stops)
+    stops = {int(s) for s in stop}
     while len(out) < max_new and out[-1] not in stops and pos < model.max_seq_len:
         if sample is None:
             burst = [int(t) for t in model.generate_greedy(out[-1], pos, min(max_new - len(out), 32, model.max_seq_len - pos))]
