@@ -402,12 +402,12 @@ def lfm2_350m_image(O, body=2, embd=14, HS=HS, IS=IS, KV=KV):
     return G.build_image(meta, tensors)
 
 
-def trace_lfm2_step(ctx, W, O, tokens=32, context=4096):
+def trace_lfm2_step(ctx, W, O, tokens=32, context=4096, **image):
     """The same decode steps enqueued one by one (no graph replay), for a kernel tracer: 32 tokens from position 1024."""
     from wick_amd import gguf as G
     from wick_amd.lfm2 import RocmLfm2Model
 
-    with G.GgufFile.from_bytes(lfm2_350m_image(O)) as g:
+    with G.GgufFile.from_bytes(lfm2_350m_image(O, **image)) as g:
         model = RocmLfm2Model(ctx, g, context)
     model.set_graph_replay(False)
     picks = model.generate_greedy(1, 1024, tokens)
@@ -415,12 +415,12 @@ def trace_lfm2_step(ctx, W, O, tokens=32, context=4096):
     return {"tokens": tokens, "start_pos": 1024, "last_pick": int(picks[-1])}
 
 
-def trace_lfm2_prefill(ctx, W, O, n=2002, context=4096):
+def trace_lfm2_prefill(ctx, W, O, n=2002, context=4096, **image):
     """One warm prompt pass of n tokens, for a kernel tracer (eager launches only)."""
     from wick_amd import gguf as G
     from wick_amd.lfm2 import RocmLfm2Model
 
-    with G.GgufFile.from_bytes(lfm2_350m_image(O)) as g:
+    with G.GgufFile.from_bytes(lfm2_350m_image(O, **image)) as g:
         model = RocmLfm2Model(ctx, g, context)
     toks = np.random.default_rng(n).integers(0, VOCAB, n)
     for _ in range(2):
@@ -775,6 +775,122 @@ def profile_figure(name, key):
     return None
 
 
+# Lokinex at the sizes of LFM2-350M / -1.2B (hidden, heads, feed-forward, vocabulary, 16 layer runs with two layers gone through
+# twice), half its layers recurrent and half attention over a cached latent; feed-forwards dense or table-routed.
+LOKINEX_SIZES = {"350m": dict(D=1024, heads=16, rank=256, dense_ff=6912, expert_ff=1024, experts=8, top=2, shared_ff=2560),
+                 "1p2b": dict(D=2048, heads=32, rank=512, dense_ff=10368, expert_ff=2048, experts=8, top=2, shared_ff=2816)}
+
+
+def lokinex_folder(path, D, heads, rank, dense_ff, expert_ff, experts, top, shared_ff, moe, vocab=VOCAB):
+    """A randomly initialised model folder (values drawn once per 4 M and repeated: the kernels' time does not depend on them)."""
+    from wick_amd.checkpoint import to_bf16, write_folder
+
+    rng = np.random.default_rng(7)
+    base = rng.standard_normal(1 << 22).astype(np.float32)
+    t = {}
+
+    def put(name, shape, sigma, center=0.0):
+        n = int(np.prod(shape))
+        t[name] = np.resize(to_bf16(center + sigma * base[:min(n, base.size)]), n).reshape(shape)
+
+    mat = lambda name, m, k: put(name, (m, k), k ** -0.5)
+    layers = []
+    for i in range(14):
+        p, x, f = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            put(p + n, (), 0.0, 1.0)
+        put(p + "canon1", (D, 4), 0.3)
+        if i % 2 == 0:
+            blocks = D // 64
+            mixer = {"type": "rglru", "mixer": {"width": D, "blocks": blocks, "conv": 4}}
+            mat(x + "y", D, D), mat(x + "x", D, D), mat(x + "o", D, D)
+            put(x + "conv", (D, 4), 0.5)
+            for n in ("y.b", "x.b", "conv.b"):
+                put(x + n, (D,), 0.1)
+            for n in ("ra", "ri"):
+                put(x + n, (blocks, 64, 64), 0.125), put(x + n + ".b", (blocks, 64), 0.3)
+            put(x + "lam", (D,), 1.0, -4.0)
+        else:
+            mixer = {"type": "latent_attention", "mixer": {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": rank, "scale": 96 ** -0.5,
+                                                           "rot": {"base": 500000.0, "dims": 32}}}
+            mat(x + "q", heads * 96, D), mat(x + "dkv", rank + 32, D), put(x + "dkv.norm", (rank,), 0.0, 1.0)
+            mat(x + "uk", heads * 64, rank), mat(x + "uv", heads * 64, rank), mat(x + "o", D, heads * 64)
+        if moe and i > 0:
+            mlp = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": shared_ff}}
+            for name, ff in [(f"e{e}", expert_ff) for e in range(experts)] + [("shared", shared_ff)]:
+                mat(f + name + ".gate", ff, D), mat(f + name + ".up", ff, D), mat(f + name + ".down", D, ff)
+            mat(f + "shared.sg", 1, D)
+            t[f + "table"] = np.argsort(rng.random((vocab, experts)), axis=1)[:, :top].astype(np.int32)
+        else:
+            mlp = {"kind": "dense", "ff": dense_ff}
+            mat(f + "up", dense_ff, D), mat(f + "down", D, dense_ff)
+        layers.append({**mixer, "mlp": mlp})
+    mat("embed", vocab, D), mat("head", vocab, D), put("final.norm", (), 0.0, 1.0)
+    mat("loop.in", D, 2 * D), put("loop.step", (2, D), 0.1)
+    write_folder(path, {"architecture": "Lokinex", "vocab": vocab, "width": D, "canon": {"taps": 4}, "norm": {"eps": 1e-6}, "layers": layers,
+                        "loop": {"start": 6, "stop": 8, "times": 2}}, t)
+
+
+def bench_lokinex(ctx, W, O, size="350m", moe=True, context=4096, tokens=64, trace=False, prompts=(512, 2002)):
+    """Decode steps and prompt passes of the Lokinex model handle, measured like bench_lfm2_step's."""
+    import tempfile
+
+    from wick_amd.model import RocmModel
+
+    with tempfile.TemporaryDirectory() as d:
+        lokinex_folder(d, moe=moe, **LOKINEX_SIZES[size])
+        model = RocmModel(ctx, d, context)
+    out = {"model": f"Lokinex {size}, {'routed' if moe else 'dense'} feed-forwards, {model.layer_runs} layer runs, bf16, random init", "context": context,
+           "gpu_memory_MB": model.gpu_memory_bytes() / 1e6, "runs": [], "prefill": []}
+    if trace:  # eager launches for a kernel tracer: 16 steps from position 1024, two prompt passes
+        model.set_graph_replay(False)
+        toks = np.random.default_rng(prompts[-1]).integers(0, VOCAB, prompts[-1])
+        for _ in range(2):
+            model.forward(toks, 0)
+        model.generate_greedy(1, 1024, 16)
+        model.free()
+        return out
+    model.generate_greedy(1, 0, 8)
+    for start in (0, 1024, context - tokens):
+        ts = []
+        for _ in range(3):
+            t0 = time.perf_counter()
+            model.generate_greedy(1, start, tokens)
+            ts.append(time.perf_counter() - t0)
+        dt = float(np.median(ts))
+        out["runs"].append({"start_pos": start, "tokens": tokens, "ms_per_token": dt / tokens * 1e3, "tokens_per_s": tokens / dt})
+    for n in prompts:
+        toks = np.random.default_rng(n).integers(0, VOCAB, n)
+        model.forward(toks, 0)
+        ts = []
+        for _ in range(7):
+            t0 = time.perf_counter()
+            model.forward(toks, 0)
+            ts.append(time.perf_counter() - t0)
+        dt = float(np.median(ts))
+        out["prefill"].append({"prompt_tokens": n, "ms": dt * 1e3, "ms_min": min(ts) * 1e3, "samples": len(ts), "tokens_per_s": n / dt})
+    ctx.kernel_timing_begin()
+    model.forward(toks, 0)
+    kt = ctx.kernel_timing_end()
+    out[f"prefill_kernel_time_{n}"] = {fam: {"us": ms * 1e3, "launches": c} for fam, (ms, c) in kt.items() if c}
+    model.set_graph_replay(False)
+    model.generate_greedy(1, 1024, 4)
+    ctx.kernel_timing_begin()
+    model.generate_greedy(1, 1028, 16)
+    kt = ctx.kernel_timing_end()
+    out["kernel_time_per_token_at_pos_1024"] = {fam: {"us": ms / 16 * 1e3, "launches": c // 16} for fam, (ms, c) in kt.items() if c}
+    model.free()
+    return out
+
+
+def bench_lokinex_all(ctx, W, O):
+    """The design beside the closest model the library had (LFM2, 8-bit blocks) at equal hidden size, heads and vocabulary."""
+    big = dict(HS=2048, IS=6912, KV=512)
+    return {"lokinex_350m": bench_lokinex(ctx, W, O, "350m"), "lokinex_350m_dense": bench_lokinex(ctx, W, O, "350m", moe=False),
+            "lfm2_350m_q8": bench_lfm2_step(ctx, W, O, body=8, embd=8), "lokinex_1p2b": bench_lokinex(ctx, W, O, "1p2b"),
+            "lfm2_1p2b_q8": bench_lfm2_step(ctx, W, O, body=8, embd=8, dims=big, label="LFM2-1.2B-shaped")}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -785,7 +901,7 @@ def main():
     ap.add_argument("--prompt-tokens", type=int, default=2002, help="lfm2_prefill_trace: tokens of the traced prompt pass")
     ap.add_argument("--graph-only", action="store_true", help="decode legs: graph replays only, no eager launches (for kernel tracers)")
     ap.add_argument("--mfma-shape", type=int, default=0, help="block loop of the wide GEMM tile: 0 / 32 (default) or 16 (A/B runs)")
-    ap.add_argument("--leg", default="all", help="all | c1 | gemm | decode | decode_q8 | gemv | prefill_sites | lm_head | lm_head_q6k | upload | lfm2_step | lfm2_step_q8 | lfm2_step_kv16 | lfm2_step_1p2b | lfm2_step_trace | lfm2_prefill_trace | copy | probe | cpu")
+    ap.add_argument("--leg", default="all", help="all | c1 | gemm | decode | decode_q8 | gemv | prefill_sites | lm_head | lm_head_q6k | upload | lfm2_step | lfm2_step_q8 | lfm2_step_kv16 | lfm2_step_1p2b | lfm2_step_trace | lfm2_prefill_trace | lokinex | lokinex_350m | lokinex_trace | lfm2_q8_trace | copy | probe | cpu")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on ONE GPU only (no collectives, no sharding); use --gpus 1", file=sys.stderr)
@@ -819,6 +935,11 @@ def main():
             "lfm2_step_1p2b": lambda: bench_lfm2_step(ctx, W, O, dims=dict(HS=2048, IS=6912, KV=512), label="LFM2-1.2B-shaped"),
             "lfm2_step_trace": lambda: trace_lfm2_step(ctx, W, O),
             "lfm2_prefill_trace": lambda: trace_lfm2_prefill(ctx, W, O, n=args.prompt_tokens),
+            # another architecture at equal sizes, and its eager launches for a kernel tracer
+            "lokinex": lambda: bench_lokinex_all(ctx, W, O),
+            "lokinex_350m": lambda: bench_lokinex(ctx, W, O, "350m"),
+            "lokinex_trace": lambda: bench_lokinex(ctx, W, O, "350m", trace=True),
+            "lfm2_q8_trace": lambda: [trace_lfm2_step(ctx, W, O, body=8, embd=8), trace_lfm2_prefill(ctx, W, O, body=8, embd=8)],
             "copy": lambda: bench_copy(ctx),
             "upload": lambda: bench_upload(ctx),
             "probe": lambda: bench_probe(ctx),

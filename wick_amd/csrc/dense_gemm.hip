@@ -335,8 +335,10 @@ hipError_t run_gemm(const DenseWeight& w, const GemmIn& in, const Epi& epi, cons
     };
     if (in.f32) return launch_kernel(L, kFamGemm, gemm_f32_kernel<Epi>, grid(64, 64), dim3(256), a, epi);
     if (g.tiles) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, Epi>, grid(128, kGroupTileRows), dim3(256), a, epi);
-    const dim3 big = grid(128, 128);
-    if (big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, Epi>, big, dim3(256), a, epi);
+    // the widest tile that leaves no CU without one (a short K is mostly epilogue: small tiles, more of them)
+    const dim3 big = grid(128, 128), tall = grid(128, 64);
+    if (w.kp > 256u && big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, Epi>, big, dim3(256), a, epi);
+    if (w.kp > 256u && tall.x * tall.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, Epi>, tall, dim3(256), a, epi);
     return launch_kernel(L, kFamGemm, gemm_bf16_kernel<2, 2, Epi>, grid(64, 64), dim3(256), a, epi);
 }
 

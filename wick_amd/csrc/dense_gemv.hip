@@ -11,6 +11,8 @@ namespace wick_rocm {
 
 namespace {
 
+typedef float v4f __attribute__((ext_vector_type(4)));
+
 constexpr uint32_t kThreads = 256;
 constexpr uint32_t kGemvMaxK = 15360;  // floats of LDS for the vector
 
@@ -31,6 +33,8 @@ __device__ __forceinline__ float dot8(uint4 w, float4 a, float4 b, float acc) {
     return fmaf(__uint_as_float(w.w & 0xffff0000u), b.w, acc);
 }
 
+__device__ __forceinline__ float dot4(v4f a, v4f b) { return (a[0] * b[0] + a[1] * b[1]) + (a[2] * b[2] + a[3] * b[3]); }
+
 __device__ __forceinline__ float block_sum_f32(float v, float* slots) {
     v = wave_sum_f32(v);
     __syncthreads();  // slots may still be read from an earlier call
@@ -42,90 +46,105 @@ __device__ __forceinline__ float block_sum_f32(float v, float* slots) {
 enum { kProVec = 0, kProRow = 1, kProRowConv = 2, kProLoop = 3 };
 
 // Fills vec[0 .. k): the vector itself, the row stage's h, or [x | 0 | x0 | 0].  All threads call it; it ends with a barrier.
-// NE: elements of a row per thread (dim <= 256 NE).
-template <int PRO, int NE>
+// A thread owns coordinates 4 t .. 4 t + 3 of every 1024: NQ vectors of four (dim <= 1024 NQ; rows are padded to 64).
+template <int PRO, int NQ>
 __device__ __forceinline__ void fill_vector(const GemvIn& in, uint32_t k, float* vec, float* slots) {
     const uint32_t tid = threadIdx.x;
     if constexpr (PRO == kProVec) {
-        for (uint32_t e = tid; e < k; e += kThreads) vec[e] = e < in.vec_len ? in.vec[e] : 0.0f;
+        for (uint32_t e = 4u * tid; e < k; e += 4u * kThreads) {
+            v4f v = {0.f, 0.f, 0.f, 0.f};
+            if (e < in.vec_len) v = *reinterpret_cast<const v4f*>(in.vec + e);
+            *reinterpret_cast<v4f*>(vec + e) = v;
+        }
         __syncthreads();
         return;
     } else {
         const RowStage& s = in.row;
         const bool first = blockIdx.x == 0;
-        float x[NE], y[NE];
+        const v4f zero = {0.f, 0.f, 0.f, 0.f};
+        v4f x[NQ], y[NQ];
 #pragma unroll
-        for (int i = 0; i < NE; i++) {
-            const uint32_t e = tid + kThreads * i;
-            x[i] = e < s.dim ? s.x[e] : 0.0f;
-            y[i] = s.y && e < s.dim ? s.y[e] : 0.0f;
+        for (int i = 0; i < NQ; i++) {
+            const uint32_t e = 4u * (tid + kThreads * i);
+            x[i] = e < s.dim ? *reinterpret_cast<const v4f*>(s.x + e) : zero;
+            y[i] = s.y && e < s.dim ? *reinterpret_cast<const v4f*>(s.y + e) : zero;
         }
         // the inputs of the earlier taps and the convolution's weights are requested before the reductions wait
         constexpr int TP = PRO == kProRowConv ? 4 : 1;  // taps kept in registers; more are read when they are used
-        float past[TP][NE], cw[TP][NE];
+        v4f past[TP][NQ], cw[TP][NQ];
         uint32_t pos = 0;
         if constexpr (PRO == kProRowConv) {
             pos = *in.d_pos;
 #pragma unroll
             for (int j = 0; j < TP; j++)
 #pragma unroll
-                for (int i = 0; i < NE; i++) {
-                    const uint32_t e = tid + kThreads * i;
+                for (int i = 0; i < NQ; i++) {
+                    const uint32_t e = 4u * (tid + kThreads * i);
                     const bool on = j < (int)s.taps && e < s.dim;
-                    cw[j][i] = on ? s.conv[(size_t)j * s.dim + e] : 0.0f;
+                    cw[j][i] = on ? *reinterpret_cast<const v4f*>(s.conv + (size_t)j * s.x_stride + e) : zero;
                     const uint32_t back = s.taps - 1u - (uint32_t)j;  // this tap's distance
-                    past[j][i] = on && back > 0 && pos >= back ? s.ring[(size_t)((pos - back) % s.taps) * s.dim + e] : 0.0f;
+                    past[j][i] = on && back > 0 && pos >= back ? *reinterpret_cast<const v4f*>(s.ring + (size_t)((pos - back) % s.taps) * s.x_stride + e) : zero;
                 }
         }
+#pragma unroll
+        for (int i = 0; i < NQ; i++)
+#pragma unroll
+            for (int c = 0; c < 4; c++)
+                if (4u * (tid + kThreads * i) + c >= s.dim) x[i][c] = y[i][c] = 0.0f;
         if (s.y) {
             float ss = 0.0f;
 #pragma unroll
-            for (int i = 0; i < NE; i++) ss += y[i] * y[i];
+            for (int i = 0; i < NQ; i++) ss += dot4(y[i], y[i]);
             const float sy = s.g_post / sqrtf(block_sum_f32(ss, slots) / (float)s.dim + s.eps);
 #pragma unroll
-            for (int i = 0; i < NE; i++) x[i] += y[i] * sy;
+            for (int i = 0; i < NQ; i++) x[i] += y[i] * sy;
         }
         if (s.x_out && first) {
 #pragma unroll
-            for (int i = 0; i < NE; i++) {
-                const uint32_t e = tid + kThreads * i;
-                if (e < s.dim) s.x_out[e] = x[i];
+            for (int i = 0; i < NQ; i++) {
+                const uint32_t e = 4u * (tid + kThreads * i);
+                if (e < s.dim) *reinterpret_cast<v4f*>(s.x_out + e) = x[i];
             }
         }
         if constexpr (PRO == kProLoop) {
 #pragma unroll
-            for (int i = 0; i < NE; i++) {
-                const uint32_t e = tid + kThreads * i;
-                if (e < s.dim) vec[e] = x[i], vec[in.x0_at + e] = in.x0[e];
+            for (int i = 0; i < NQ; i++) {
+                const uint32_t e = 4u * (tid + kThreads * i);
+                if (e >= in.x0_at) continue;
+                v4f v = e < s.dim ? *reinterpret_cast<const v4f*>(in.x0 + e) : zero;
+#pragma unroll
+                for (int c = 0; c < 4; c++)
+                    if (e + c >= s.dim) v[c] = 0.0f;
+                *reinterpret_cast<v4f*>(vec + e) = x[i];
+                *reinterpret_cast<v4f*>(vec + in.x0_at + e) = v;
             }
-            for (uint32_t e = s.dim + tid; e < in.x0_at; e += kThreads) vec[e] = 0.0f;
-            for (uint32_t e = in.x0_at + s.dim + tid; e < k; e += kThreads) vec[e] = 0.0f;
         } else {
             float ss = 0.0f;
 #pragma unroll
-            for (int i = 0; i < NE; i++) ss += x[i] * x[i];
+            for (int i = 0; i < NQ; i++) ss += dot4(x[i], x[i]);
             const float sx = s.g_pre / sqrtf(block_sum_f32(ss, slots) / (float)s.dim + s.eps);
 #pragma unroll
-            for (int i = 0; i < NE; i++) {
-                const uint32_t e = tid + kThreads * i;
-                if (e >= s.dim) continue;
-                float h = x[i] * sx;
+            for (int i = 0; i < NQ; i++) {
+                const uint32_t e = 4u * (tid + kThreads * i);
+                if (e >= k) continue;
+                v4f h = x[i] * sx;
                 if constexpr (PRO == kProRowConv) {
-                    if (first) s.ring[(size_t)(pos % s.taps) * s.dim + e] = h;
-                    float c = 0.0f;
+                    if (e < s.dim) {
+                        if (first) *reinterpret_cast<v4f*>(s.ring + (size_t)(pos % s.taps) * s.x_stride + e) = h;
+                        v4f c = zero;
 #pragma unroll
-                    for (int j = 0; j < TP; j++)
-                        if (j < (int)s.taps) c += cw[j][i] * (j + 1 == (int)s.taps ? h : past[j][i]);
-                    for (uint32_t j = TP; j < s.taps; j++) {
-                        const uint32_t back = s.taps - 1u - j;
-                        const float v = back == 0 ? h : pos >= back ? s.ring[(size_t)((pos - back) % s.taps) * s.dim + e] : 0.0f;
-                        c += s.conv[(size_t)j * s.dim + e] * v;
+                        for (int j = 0; j < TP; j++)
+                            if (j < (int)s.taps) c += cw[j][i] * (j + 1 == (int)s.taps ? h : past[j][i]);
+                        for (uint32_t j = TP; j < s.taps; j++) {
+                            const uint32_t back = s.taps - 1u - j;
+                            const v4f v = back == 0 ? h : pos >= back ? *reinterpret_cast<const v4f*>(s.ring + (size_t)((pos - back) % s.taps) * s.x_stride + e) : zero;
+                            c += *reinterpret_cast<const v4f*>(s.conv + (size_t)j * s.x_stride + e) * v;
+                        }
+                        h += c;  // (zero past dim: so are the inputs there and the weights)
                     }
-                    h += c;
                 }
-                vec[e] = h;
+                *reinterpret_cast<v4f*>(vec + e) = h;
             }
-            for (uint32_t e = s.dim + tid; e < k; e += kThreads) vec[e] = 0.0f;
         }
         __syncthreads();
     }
@@ -180,7 +199,7 @@ struct DenseArgs {
     uint32_t split;
 };
 
-template <int PRO, int NE, int R>
+template <int PRO, int NQ, int R>
 __global__ __launch_bounds__(256) void gemv_dense_kernel(DenseArgs a) {
     extern __shared__ __align__(16) float vec[];
     __shared__ float slots[4];
@@ -190,7 +209,7 @@ __global__ __launch_bounds__(256) void gemv_dense_kernel(DenseArgs a) {
     for (int r = 0; r < R; r++) rows[r] = a.w + (size_t)(row0 + r < a.m ? row0 + r : a.m - 1u) * a.ldw;
     Ahead<R> ahead;
     ahead.load(rows, a.k);
-    fill_vector<PRO, NE>(a.in, a.k, vec, slots);
+    fill_vector<PRO, NQ>(a.in, a.k, vec, slots);
     float acc[R];
 #pragma unroll
     for (int r = 0; r < R; r++) acc[r] = 0.0f;
@@ -218,7 +237,7 @@ struct RoutedArgs {
 
 __device__ __forceinline__ uint32_t routed_expert(const RoutedArgs& a, uint32_t s) { return (uint32_t)a.m.table[(size_t)*a.d_token * a.m.top + s]; }
 
-template <int NE, int R>
+template <int NQ, int R>
 __global__ __launch_bounds__(256) void gemv_routed_up_kernel(RoutedArgs a) {
     extern __shared__ __align__(16) float vec[];
     __shared__ float slots[4];
@@ -244,7 +263,7 @@ __global__ __launch_bounds__(256) void gemv_routed_up_kernel(RoutedArgs a) {
     }
     Ahead<2 * R> ahead;
     ahead.load(rows, a.k);
-    fill_vector<kProRow, NE>(a.in, a.k, vec, slots);
+    fill_vector<kProRow, NQ>(a.in, a.k, vec, slots);
     if (f0 > total || (f0 == total && !shared)) return;
     float acc[2 * R];
 #pragma unroll
@@ -262,29 +281,50 @@ __global__ __launch_bounds__(256) void gemv_routed_up_kernel(RoutedArgs a) {
     }
 }
 
+// The experts' rows and the shared one's are one long row over the concatenated activations.  All pieces a wave needs of it (up to
+// kDownAhead of 512 columns) are requested before the activations are scaled into LDS.
+constexpr int kDownAhead = 10;
+
 template <int R>
 __global__ __launch_bounds__(256) void gemv_routed_down_kernel(RoutedArgs a) {
     extern __shared__ __align__(16) float vec[];
     const RoutedMlp& m = a.m;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, row0 = (blockIdx.x * 4u + (tid >> 6)) * R;
     const uint32_t ff = m.down.kp, routed = m.top * ff, shared = m.shared_down.d ? m.shared_down.kp : 0u, total = routed + shared;
+    const int32_t* chosen = m.table + (size_t)*a.d_token * m.top;
+    auto piece = [&](uint32_t at, uint32_t r) {  // 8 weights of row r from column `at` (segments are multiples of 64 columns)
+        const uint32_t row = row0 + r < a.rows ? row0 + r : a.rows - 1u;
+        if (at >= total) return uint4{0, 0, 0, 0};
+        const uint16_t* p = at < routed ? m.down.d + (size_t)chosen[at / ff] * m.down.stride + (size_t)row * ff + at % ff
+                                        : m.shared_down.d + (size_t)row * shared + (at - routed);
+        return *reinterpret_cast<const uint4*>(p);
+    };
+    uint4 w[kDownAhead][R];
+#pragma unroll
+    for (int c = 0; c < kDownAhead; c++)
+#pragma unroll
+        for (int r = 0; r < R; r++) w[c][r] = piece(512u * c + 8u * lane, r);
     const float share = 1.0f / (float)m.top, gate = shared ? a.act_in[total] : 0.0f;
-    for (uint32_t e = tid; e < total; e += kThreads) vec[e] = a.act_in[e] * (e < routed ? share : gate);
+    for (uint32_t e = 4u * tid; e < total; e += 4u * kThreads) {
+        const v4f v = *reinterpret_cast<const v4f*>(a.act_in + e);
+        *reinterpret_cast<v4f*>(vec + e) = v * (e < routed ? share : gate);
+    }
     __syncthreads();
     float acc[R];
 #pragma unroll
     for (int r = 0; r < R; r++) acc[r] = 0.0f;
-    const uint16_t* rows[R];
-    for (uint32_t s = 0; s < m.top; s++) {
-        const uint16_t* base = m.down.d + (size_t)routed_expert(a, s) * m.down.stride;
 #pragma unroll
-        for (int r = 0; r < R; r++) rows[r] = base + (size_t)(row0 + r < a.rows ? row0 + r : a.rows - 1u) * ff;
-        dot_rows<R, false>(rows, nullptr, vec + s * ff, ff, acc);
+    for (int c = 0; c < kDownAhead; c++) {
+        const uint32_t at = 512u * c + 8u * lane;
+        if (at >= total) break;
+        const float4 v0 = *reinterpret_cast<const float4*>(vec + at), v1 = *reinterpret_cast<const float4*>(vec + at + 4);
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = dot8(w[c][r], v0, v1, acc[r]);
     }
-    if (shared) {
+    for (uint32_t at = 512u * kDownAhead + 8u * lane; at < total; at += 512u) {
+        const float4 v0 = *reinterpret_cast<const float4*>(vec + at), v1 = *reinterpret_cast<const float4*>(vec + at + 4);
 #pragma unroll
-        for (int r = 0; r < R; r++) rows[r] = m.shared_down.d + (size_t)(row0 + r < a.rows ? row0 + r : a.rows - 1u) * shared;
-        dot_rows<R, false>(rows, nullptr, vec + routed, shared, acc);
+        for (int r = 0; r < R; r++) acc[r] = dot8(piece(at, r), v0, v1, acc[r]);
     }
 #pragma unroll
     for (int r = 0; r < R; r++) {
@@ -293,26 +333,26 @@ __global__ __launch_bounds__(256) void gemv_routed_down_kernel(RoutedArgs a) {
     }
 }
 
-template <int PRO, int NE>
+template <int PRO, int NQ>
 hipError_t run_dense(const DenseArgs& a, const Launch& L) {
     const uint32_t lds = a.k * 4u;
-    if (a.m <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NE, 1>, dim3((a.m + 3u) / 4u), dim3(kThreads), lds, a);
-    if (a.m <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NE, 2>, dim3((a.m + 7u) / 8u), dim3(kThreads), lds, a);
-    return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NE, 4>, dim3((a.m + 15u) / 16u), dim3(kThreads), lds, a);
+    if (a.m <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NQ, 1>, dim3((a.m + 3u) / 4u), dim3(kThreads), lds, a);
+    if (a.m <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NQ, 2>, dim3((a.m + 7u) / 8u), dim3(kThreads), lds, a);
+    return launch_kernel_lds(L, kFamGemv, gemv_dense_kernel<PRO, NQ, 4>, dim3((a.m + 15u) / 16u), dim3(kThreads), lds, a);
 }
 
 template <int PRO>
-hipError_t run_dense_ne(const DenseArgs& a, const Launch& L) {
+hipError_t run_dense_nq(const DenseArgs& a, const Launch& L) {
     const uint32_t dim = a.in.row.dim;
-    if (dim <= 1024u) return run_dense<PRO, 4>(a, L);
-    if (dim <= 2048u) return run_dense<PRO, 8>(a, L);
-    if (dim <= 4096u) return run_dense<PRO, 16>(a, L);
-    if (dim <= 8192u) return run_dense<PRO, 32>(a, L);
+    if (dim <= 1024u) return run_dense<PRO, 1>(a, L);
+    if (dim <= 2048u) return run_dense<PRO, 2>(a, L);
+    if (dim <= 4096u) return run_dense<PRO, 4>(a, L);
+    if (dim <= 8192u) return run_dense<PRO, 8>(a, L);
     return hipErrorInvalidValue;
 }
 
 bool row_ok(const RowStage& s, uint32_t k) {
-    return s.x && s.dim > 0 && s.dim <= k && s.x_out != s.x && (!s.conv || (s.ring && s.taps > 0)) && !s.experts;
+    return s.x && s.dim > 0 && pad_to(s.dim, 4) <= s.x_stride && s.x_stride % 4u == 0 && k <= pad_to(s.dim, kDensePad) * 2u && s.dim <= k && s.x_out != s.x && (!s.conv || (s.ring && s.taps > 0)) && !s.experts;
 }
 
 }  // namespace
@@ -322,14 +362,15 @@ hipError_t launch_gemv_dense(const DenseWeight& w, uint32_t m, const GemvIn& in,
     if (!w.d || !out || m == 0 || m > w.mp || a.k > w.kp || a.k % 8u || a.k > kGemvMaxK || w.kp % 8u) return hipErrorInvalidValue;
     if (in.vec) {
         if (a.in.vec_len == 0) a.in.vec_len = a.k;
+        if (a.in.vec_len % 4u) return hipErrorInvalidValue;
         return run_dense<kProVec, 1>(a, L);
     }
     if (!row_ok(in.row, a.k) || (in.row.conv && !in.d_pos)) return hipErrorInvalidValue;
     if (in.x0) {
-        if (in.x0_at < in.row.dim || in.x0_at + in.row.dim > a.k) return hipErrorInvalidValue;
-        return run_dense_ne<kProLoop>(a, L);
+        if (in.x0_at != pad_to(in.row.dim, kDensePad) || 2u * in.x0_at != a.k) return hipErrorInvalidValue;
+        return run_dense_nq<kProLoop>(a, L);
     }
-    return in.row.conv ? run_dense_ne<kProRowConv>(a, L) : run_dense_ne<kProRow>(a, L);
+    return in.row.conv ? run_dense_nq<kProRowConv>(a, L) : run_dense_nq<kProRow>(a, L);
 }
 
 uint32_t routed_act_floats(const RoutedMlp& m) { return m.top * (m.gate_up.mp / 2u) + (m.shared_gate_up.d ? m.shared_gate_up.mp / 2u : 0u) + 4u; }
@@ -344,10 +385,10 @@ hipError_t launch_gemv_routed_up(const RoutedMlp& m, const GemvIn& in, const uin
     const uint32_t features = routed_act_floats(m) - 4u, waves = features / R + 1u;
     const dim3 grid((waves + 3u) / 4u);
     const uint32_t lds = a.k * 4u, dim = in.row.dim;
-    if (dim <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<4, R>, grid, dim3(kThreads), lds, a);
-    if (dim <= 2048u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<8, R>, grid, dim3(kThreads), lds, a);
-    if (dim <= 4096u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<16, R>, grid, dim3(kThreads), lds, a);
-    if (dim <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<32, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<1, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 2048u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<2, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 4096u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<4, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_routed_up_kernel<8, R>, grid, dim3(kThreads), lds, a);
     return hipErrorInvalidValue;
 }
 

@@ -21,6 +21,7 @@ typedef uint32_t u4 __attribute__((ext_vector_type(4)));
 constexpr uint32_t kChunk = 64;      // positions per pass
 constexpr uint32_t kMaxSplits = 64;  // workgroups along the sequence
 constexpr uint32_t kSlab = 128;      // latent columns per workgroup of the absorbing launch
+constexpr uint32_t kStageBytes = 144u * 1024u;  // dynamic LDS of the staged form, beside its static 6 KB
 constexpr float kLog2e = 1.44269504088896340736f;
 
 __device__ __forceinline__ void put(float* p, float v) { *p = v; }
@@ -162,11 +163,13 @@ __device__ __forceinline__ void load8(const CT* p, float (&v)[8]) {
     }
 }
 
-// Workgroup (split, HG heads, token).  Scores: 16 lanes walk the pieces of four cache rows at a time, so a piece of a query is read
-// from LDS once for four positions.  Values: a thread owns NP pairs of latent columns for all HG heads.
-template <int HG, int NP, typename CT>
+// Workgroup (split, HG heads, token).  STAGED: a chunk's cache rows are brought into LDS once (all of a thread's loads in flight
+// together) and serve both halves; rows too long for that are read from memory twice.  Scores: 16 lanes walk the pieces of four
+// cache rows at a time, so a piece of a query is read from LDS once for four positions.  Values: a thread owns NP pairs of latent
+// columns for all HG heads.
+template <int HG, int NP, bool STAGED, typename CT>
 __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
-    extern __shared__ __align__(16) float qs[];  // [HG][row]
+    extern __shared__ __align__(16) float qs[];  // [HG][row], then STAGED: [kChunk][row] of the cache type
     __shared__ __align__(16) float sc[HG][kChunk], wt[kChunk][HG];
     __shared__ float corr[HG];
     __shared__ float red[256 * 2];
@@ -197,9 +200,25 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
 
     for (uint32_t c = split; c * kChunk <= pos; c += a.splits) {
         const uint32_t t0 = c * kChunk, nt = pos + 1u - t0 < kChunk ? pos + 1u - t0 : kChunk;
+        const CT* rows = cache + (size_t)t0 * row;
+        if constexpr (STAGED) {
+            constexpr uint32_t PER = 16 / sizeof(CT);
+            CT* stage = reinterpret_cast<CT*>(qs + HG * row);
+            const uint32_t pieces = nt * (row / PER);
+            for (uint32_t i0 = tid; i0 < pieces; i0 += 8u * 256u) {
+                u4 v[8];
+#pragma unroll
+                for (int j = 0; j < 8; j++) v[j] = *reinterpret_cast<const u4*>(rows + (size_t)(i0 + 256u * j < pieces ? i0 + 256u * j : i0) * PER);
+#pragma unroll
+                for (int j = 0; j < 8; j++)
+                    if (i0 + 256u * j < pieces) *reinterpret_cast<u4*>(stage + (size_t)(i0 + 256u * j) * PER) = v[j];
+            }
+            rows = stage;
+            __syncthreads();
+        }
         const CT* kr[4];
 #pragma unroll
-        for (int k = 0; k < 4; k++) kr[k] = cache + (size_t)(t0 + (key_in + k < nt ? key_in + k : nt - 1u)) * row;
+        for (int k = 0; k < 4; k++) kr[k] = rows + (size_t)(key_in + k < nt ? key_in + k : nt - 1u) * row;
         float dot[4][HG];
 #pragma unroll
         for (int k = 0; k < 4; k++)
@@ -248,9 +267,9 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
             for (int i = 0; i < NP; i++) acc[i][h][0] *= f, acc[i][h][1] *= f;
         }
         if (cp < pairs) {
-#pragma unroll 4
+#pragma unroll 8
             for (uint32_t k = kg; k < nt; k += kgroups) {
-                const CT* vr = cache + (size_t)(t0 + k) * row;
+                const CT* vr = rows + (size_t)k * row;
                 float w[HG];
 #pragma unroll
                 for (int h = 0; h < HG; h++) w[h] = wt[k][h];
@@ -312,6 +331,14 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
     const uint32_t h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x, lane = tid & 63u;
     const uint32_t pos = (a.d_pos ? *a.d_pos : a.pos0) + t;
     if (pos >= s.max_seq) return;
+    // the first four value rows of a wave are requested before the partials are looked at (rank_p <= 512: whole rows)
+    const uint32_t waves = gridDim.z * 4u, first = blockIdx.z * 4u + (tid >> 6);
+    float ahead[4][8];
+#pragma unroll
+    for (int r = 0; r < 4; r++) {
+        const uint32_t v = first + r * waves < s.vdim ? first + r * waves : s.vdim - 1u;
+        if (8u * lane < s.rank_p) load8(a.uv + ((size_t)h * s.vdim + v) * s.rank_p + 8u * lane, ahead[r]);
+    }
     uint32_t active = pos / kChunk + 1u;
     active = active < a.splits ? active : a.splits;
     const uint32_t stride = s.rank_p + 4u;
@@ -336,8 +363,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
     }
     __syncthreads();
     OT* out = static_cast<OT*>(a.out) + (size_t)t * a.ldo;
-    const uint32_t waves = gridDim.z * 4u;
-    for (uint32_t v0 = blockIdx.z * 4u + (tid >> 6); v0 < s.vdim; v0 += 4u * waves) {
+    for (uint32_t v0 = first; v0 < s.vdim; v0 += 4u * waves) {
         float d[4] = {0.f, 0.f, 0.f, 0.f};
         for (uint32_t at = 8u * lane; at < s.rank_p; at += 512u) {
             const v4f o0 = *reinterpret_cast<const v4f*>(oc + at), o1 = *reinterpret_cast<const v4f*>(oc + at + 4);
@@ -345,7 +371,12 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
             for (int r = 0; r < 4; r++) {
                 const uint32_t v = v0 + r * waves < s.vdim ? v0 + r * waves : v0;
                 float w[8];
-                load8(a.uv + ((size_t)h * s.vdim + v) * s.rank_p + at, w);
+                if (v0 == first && at < 512u) {
+#pragma unroll
+                    for (int i = 0; i < 8; i++) w[i] = ahead[r][i];
+                } else {
+                    load8(a.uv + ((size_t)h * s.vdim + v) * s.rank_p + at, w);
+                }
 #pragma unroll
                 for (int i = 0; i < 4; i++) d[r] = fmaf(w[i], o0[i], fmaf(w[4 + i], o1[i], d[r]));
             }
@@ -553,9 +584,19 @@ hipError_t launch_latent_attention(const LatentShape& s, const LatentWeights& w,
     auto attend = [&](auto hg, auto np) {
         constexpr int HG = decltype(hg)::value, NP = decltype(np)::value;
         const dim3 grid(splits, (s.heads + HG - 1u) / HG, n);
-        const uint32_t lds = HG * s.row() * 4u;
-        return s.f32 ? launch_kernel_lds(L, kFamOther, latent_attend_kernel<HG, NP, float>, grid, dim3(256), lds, a)
-                     : launch_kernel_lds(L, kFamOther, latent_attend_kernel<HG, NP, uint16_t>, grid, dim3(256), lds, a);
+        const uint32_t lds = HG * s.row() * 4u, staged = lds + kChunk * s.row() * (s.f32 ? 4u : 2u);
+        if constexpr (NP <= 2) {  // (longer rows do not fit)
+            auto go = [&](auto kernel) {
+                if (staged > 56u * 1024u) {
+                    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kStageBytes);
+                    if (e != hipSuccess) return e;
+                }
+                return launch_kernel_lds(L, kFamOther, kernel, grid, dim3(256), staged, a);
+            };
+            if (staged <= kStageBytes) return s.f32 ? go(latent_attend_kernel<HG, NP, true, float>) : go(latent_attend_kernel<HG, NP, true, uint16_t>);
+        }
+        return s.f32 ? launch_kernel_lds(L, kFamOther, latent_attend_kernel<HG, NP, false, float>, grid, dim3(256), lds, a)
+                     : launch_kernel_lds(L, kFamOther, latent_attend_kernel<HG, NP, false, uint16_t>, grid, dim3(256), lds, a);
     };
     auto with_pairs = [&](auto hg) {
         if (s.rank_p <= 512u) return attend(hg, std::integral_constant<int, 1>{});

@@ -46,7 +46,7 @@ struct Layer {
     MixerConfig mix;
     MlpConfig mlp;
     float norm1 = 0, norm1b = 0, norm2 = 0, norm2b = 0;
-    float* canon = nullptr;   // [taps][width]
+    float* canon = nullptr;   // [taps][dp]
     DenseWeight in, out;
     // rglru: channels in blocks padded to `block`
     uint32_t block = 0, channels = 0;
@@ -316,9 +316,9 @@ int Lokinex::load_layer(wick_rocm_ctx* ctx, const wick_safetensors* f, uint32_t 
     l.norm1 = scalar(f, p + "norm1"), l.norm1b = scalar(f, p + "norm1b");
     {
         const uint16_t* w = tensor(f, p + "canon1", {D, cfg.taps});
-        std::vector<float> v((size_t)cfg.taps * D);
+        std::vector<float> v((size_t)cfg.taps * dp, 0.0f);
         for (uint32_t e = 0; e < D; e++)
-            for (uint32_t k = 0; k < cfg.taps; k++) v[(size_t)k * D + e] = bf16(w[(size_t)e * cfg.taps + k]);
+            for (uint32_t k = 0; k < cfg.taps; k++) v[(size_t)k * dp + e] = bf16(w[(size_t)e * cfg.taps + k]);
         LK_TRY(upload(ctx, this, v, &l.canon));
     }
     if (m.recurrent) {
@@ -487,7 +487,7 @@ int Lokinex::load(wick_rocm_ctx* ctx, const wick_safetensors* f, uint32_t contex
         const MixerConfig& m = l.first;
         const MlpConfig& c = l.second;
         const uint64_t routed = (uint64_t)c.top * pad_to(c.ff, kDensePad) + pad_to(c.shared_ff, kDensePad);
-        const bool ok = m.recurrent ? (uint64_t)m.blocks * pad_to(m.width / m.blocks, kDensePad) <= 15360u && m.width / m.blocks <= 4096u && m.conv <= 16u
+        const bool ok = m.recurrent ? (uint64_t)m.blocks * pad_to(m.width / m.blocks, kDensePad) <= 15360u && m.width / m.blocks <= 4096u && m.conv <= 8u
                                     : (uint64_t)m.heads * m.vdim <= 15360u && m.rank <= 2048u && m.rot <= 1024u && (uint64_t)m.heads * (m.dim + m.rot) <= 1u << 20;
         if (!ok || (c.kind == MlpConfig::kDense && c.ff > 15360u) || (c.kind == MlpConfig::kMoe && (routed > 15360u || c.experts > kRouteMaxExperts)))
             throw ConfigError{"a layer's sizes are beyond what the kernels take"};
@@ -537,7 +537,7 @@ int Lokinex::load(wick_rocm_ctx* ctx, const wick_safetensors* f, uint32_t contex
     size_t scratch_w = 4;
     for (Run& r : runs) {
         const Layer& l = layers[r.layer];
-        LK_TRY(alloc_t(ctx, (size_t)cfg.taps * D, &r.canon_ring));
+        LK_TRY(alloc_t(ctx, (size_t)cfg.taps * dp, &r.canon_ring));
         proj_w = std::max(proj_w, l.in.mp), mixed_w = std::max(mixed_w, l.out.kp);
         if (l.mix.recurrent) {
             LK_TRY(alloc_t(ctx, (size_t)l.mix.conv * l.channels, &r.conv_ring));
@@ -914,7 +914,7 @@ template <typename F>
 int Lokinex::for_each_state_piece(uint32_t seq_len, F&& piece) const {
     for (const Run& r : runs) {
         const Layer& l = layers[r.layer];
-        LK_TRY(piece(r.canon_ring, (size_t)cfg.taps * cfg.width * sizeof(float)));
+        LK_TRY(piece(r.canon_ring, (size_t)cfg.taps * dp * sizeof(float)));
         if (l.mix.recurrent) {
             LK_TRY(piece(r.conv_ring, (size_t)l.mix.conv * l.channels * sizeof(float)));
             LK_TRY(piece(r.state, (size_t)l.channels * sizeof(float)));

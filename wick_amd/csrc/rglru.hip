@@ -11,36 +11,40 @@ namespace wick_rocm {
 
 namespace {
 
-constexpr uint32_t kConvTokens = 16;   // tokens per thread of the prompt convolution; at least taps - 1
+constexpr uint32_t kConvTokens = 8;    // tokens per thread of the prompt convolution; at least taps - 1
 constexpr uint32_t kScanChunk = 32;
 
 __device__ __forceinline__ void put(float* p, float v) { *p = v; }
 __device__ __forceinline__ void put(uint16_t* p, float v) { *p = __builtin_bit_cast(uint16_t, (__bf16)v); }
 
-// One thread: one channel, kConvTokens tokens.  Only the threads of the first tokens read the ring, and they alone write it, after
-// their reads.
-template <typename AT>
+// One thread: one channel, kConvTokens tokens, their inputs and the ones in front of them in registers (FAST: up to four taps).
+// Only the threads of the first tokens read the ring, and they alone write it, after their reads.
+template <bool FAST, typename AT>
 __global__ __launch_bounds__(256) void recurrent_conv_kernel(RecurrentConv a, uint32_t n) {
+    constexpr int BACK = FAST ? 3 : (int)kConvTokens;
     const uint32_t ch = blockIdx.x * 256u + threadIdx.x, t0 = blockIdx.y * kConvTokens;
     if (ch >= a.channels) return;
     const float* x = a.proj + a.x_at + ch;
     const uint32_t block = ch / a.block, terms = sizeof(AT) == 2 ? 2u : 1u;
     AT* ua = static_cast<AT*>(a.ua) + (size_t)block * terms * a.block + ch % a.block;
     const float bias = a.bias[ch];
-    const uint32_t t1 = t0 + kConvTokens < n ? t0 + kConvTokens : n;
-    for (uint32_t t = t0; t < t1; t++) {
+    float in[BACK + (int)kConvTokens], w[BACK + 1];  // w by distance: the newest input is the last tap
+#pragma unroll
+    for (int i = 0; i < BACK + (int)kConvTokens; i++) {
+        const int t = (int)t0 + i - BACK, p = (int)a.pos0 + t;
+        in[i] = 0.0f;
+        if (t >= 0) in[i] = x[(size_t)(t < (int)n ? t : (int)n - 1) * a.ldp];
+        else if (p >= 0 && BACK - i < (int)a.taps) in[i] = a.ring[(size_t)((uint32_t)p % a.taps) * a.channels + ch];
+    }
+#pragma unroll
+    for (int m = 0; m <= BACK; m++) w[m] = m < (int)a.taps ? a.w[(size_t)(a.taps - 1u - m) * a.channels + ch] : 0.0f;
+#pragma unroll
+    for (int i = 0; i < (int)kConvTokens; i++) {
+        const uint32_t t = t0 + i;
+        if (t >= n) break;
         float v = 0.0f;
-        for (uint32_t k = 0; k < a.taps; k++) {
-            const int src = (int)(t + k) - (int)(a.taps - 1u);
-            float tap = 0.0f;
-            if (src >= 0) {
-                tap = x[(size_t)src * a.ldp];
-            } else {
-                const int p = (int)a.pos0 + src;
-                if (p >= 0) tap = a.ring[(size_t)((uint32_t)p % a.taps) * a.channels + ch];
-            }
-            v += a.w[(size_t)k * a.channels + ch] * tap;
-        }
+#pragma unroll
+        for (int m = BACK; m >= 0; m--) v += w[m] * in[i + BACK - m];
         v += bias;
         a.u[(size_t)t * a.channels + ch] = v;
         AT* o = ua + (size_t)t * a.lda;
@@ -67,15 +71,15 @@ __global__ __launch_bounds__(256) void scan_chunks_kernel(const float* __restric
         scratch[(size_t)2 * chunks * channels + ch] = s;
     }
     const uint32_t t0 = c * kScanChunk, nt = n - t0 < kScanChunk ? n - t0 : kScanChunk;
-    for (uint32_t i = 0; i < nt; i += 8) {
-        float av[8], bv[8];
+    for (uint32_t i = 0; i < nt; i += 16) {
+        float av[16], bv[16];
 #pragma unroll
-        for (int j = 0; j < 8; j++) {
+        for (int j = 0; j < 16; j++) {
             const size_t at = (size_t)(t0 + (i + j < nt ? i + j : nt - 1u)) * channels + ch;
             av[j] = a[at], bv[j] = b[at];
         }
 #pragma unroll
-        for (int j = 0; j < 8; j++)
+        for (int j = 0; j < 16; j++)
             if (i + j < nt) prod *= av[j], s = av[j] * s + bv[j];
     }
     scratch[(size_t)c * channels + ch] = prod;
@@ -105,15 +109,15 @@ __global__ __launch_bounds__(256) void scan_apply_kernel(const float* __restrict
         for (int j = 0; j < 8; j++)
             if (q0 + j < c) s = av[j] * s + bv[j];
     }
-    for (uint32_t i = 0; i < nt; i += 8) {
-        float av[8], bv[8], yv[8];
+    for (uint32_t i = 0; i < nt; i += 16) {
+        float av[16], bv[16], yv[16];
 #pragma unroll
-        for (int j = 0; j < 8; j++) {
+        for (int j = 0; j < 16; j++) {
             const uint32_t t = t0 + (i + j < nt ? i + j : nt - 1u);
             av[j] = a[(size_t)t * channels + ch], bv[j] = b[(size_t)t * channels + ch], yv[j] = y[(size_t)t * ldy + ch];
         }
 #pragma unroll
-        for (int j = 0; j < 8; j++)
+        for (int j = 0; j < 16; j++)
             if (i + j < nt) {
                 s = av[j] * s + bv[j];
                 put(out + (size_t)(t0 + i + j) * ldo + ch, s * yv[j]);
@@ -133,6 +137,12 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(RecurrentStep a) {
     const uint32_t parts = a.block / kStepPart, blk = blockIdx.x / parts, part = blockIdx.x % parts;
     const uint32_t tid = threadIdx.x, pos = *a.d_pos, c0 = blk * a.block;
     const uint32_t l = tid % LPR, grp = tid / LPR;
+    const uint16_t* w = a.gates.d + (size_t)blk * a.gates.stride;
+    auto row_of = [&](uint32_t f) { return w + (size_t)((f >> 4) * 32u + (f & 15u)) * a.gates.kp; };
+    // requested before the convolution whose result they meet
+    const uint16_t* row0 = row_of(part * kStepPart + grp);
+    const uint32_t at0 = 8u * l < a.block ? 8u * l : 0u;
+    const uint4 q0 = *reinterpret_cast<const uint4*>(row0 + at0), p0 = *reinterpret_cast<const uint4*>(row0 + (size_t)16 * a.gates.kp + at0);
     for (uint32_t i = tid; i < a.block; i += 256) {
         const uint32_t ch = c0 + i;
         const float now = a.proj[a.channels + ch];
@@ -147,14 +157,14 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(RecurrentStep a) {
         if (part == 0) a.ring[(size_t)(pos % a.taps) * a.channels + ch] = now;
     }
     __syncthreads();
-    const uint16_t* w = a.gates.d + (size_t)blk * a.gates.stride;
     for (uint32_t f0 = 0; f0 < kStepPart; f0 += 256u / LPR) {
         const uint32_t f = part * kStepPart + f0 + grp;  // channel of the block; LPR >= 8: a pass covers at most kStepPart channels
-        const uint16_t* rw = w + (size_t)((f >> 4) * 32u + (f & 15u)) * a.gates.kp;
+        const uint16_t* rw = row_of(f);
         const uint16_t* iw = rw + (size_t)16 * a.gates.kp;
         float r = 0.0f, g = 0.0f;
         for (uint32_t at = 8u * l; at < a.block; at += 8u * LPR) {
-            const uint4 q = *reinterpret_cast<const uint4*>(rw + at), p = *reinterpret_cast<const uint4*>(iw + at);
+            const bool first = f0 == 0 && at == 8u * l;
+            const uint4 q = first ? q0 : *reinterpret_cast<const uint4*>(rw + at), p = first ? p0 : *reinterpret_cast<const uint4*>(iw + at);
             const uint32_t qv[4] = {q.x, q.y, q.z, q.w}, pv[4] = {p.x, p.y, p.z, p.w};
 #pragma unroll
             for (int k = 0; k < 4; k++) {
@@ -178,10 +188,14 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(RecurrentStep a) {
 
 hipError_t launch_recurrent_conv(const RecurrentConv& a, uint32_t n, const Launch& L) {
     if (n == 0) return hipSuccess;
-    if (a.taps == 0 || a.taps - 1u > kConvTokens || a.block == 0 || a.channels % a.block || a.lda < a.channels * (a.f32 ? 1u : 2u)) return hipErrorInvalidValue;
+    if (a.taps == 0 || a.taps > kConvTokens || a.block == 0 || a.channels % a.block || a.lda < a.channels * (a.f32 ? 1u : 2u)) return hipErrorInvalidValue;
     const dim3 grid((a.channels + 255u) / 256u, (n + kConvTokens - 1u) / kConvTokens);
-    return a.f32 ? launch_kernel(L, kFamOther, recurrent_conv_kernel<float>, grid, dim3(256), a, n)
-                 : launch_kernel(L, kFamOther, recurrent_conv_kernel<uint16_t>, grid, dim3(256), a, n);
+    auto go = [&](auto fast) {
+        constexpr bool F = decltype(fast)::value;
+        return a.f32 ? launch_kernel(L, kFamOther, recurrent_conv_kernel<F, float>, grid, dim3(256), a, n)
+                     : launch_kernel(L, kFamOther, recurrent_conv_kernel<F, uint16_t>, grid, dim3(256), a, n);
+    };
+    return a.taps <= 4u ? go(std::integral_constant<bool, true>{}) : go(std::integral_constant<bool, false>{});
 }
 
 size_t recurrent_scan_scratch_floats(uint32_t n, uint32_t channels) { return ((size_t)2 * ((n + kScanChunk - 1u) / kScanChunk) + 1u) * channels; }

@@ -7,10 +7,21 @@ namespace wick_rocm {
 
 namespace {
 
+typedef float v4f __attribute__((ext_vector_type(4)));
+typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+
 constexpr uint32_t kRowsLdsBytes = 160u * 1024u;
 
 __device__ __forceinline__ void put(float* p, float v) { *p = v; }
 __device__ __forceinline__ void put(uint16_t* p, float v) { *p = __builtin_bit_cast(uint16_t, (__bf16)v); }
+
+__device__ __forceinline__ void store4(float* p, v4f v) { *reinterpret_cast<v4f*>(p) = v; }
+__device__ __forceinline__ void store4(uint16_t* p, v4f v) {
+    bf4 b;
+#pragma unroll
+    for (int i = 0; i < 4; i++) b[i] = (__bf16)v[i];
+    *reinterpret_cast<bf4*>(p) = b;
+}
 
 // y of token t at coordinate e: the sublayer's output, or the mean of the routed experts' outputs on top of it.
 __device__ __forceinline__ float row_y(const RowStage& s, uint32_t t, uint32_t e) {
@@ -52,7 +63,7 @@ __device__ __forceinline__ void stage_row(const RowStage& s, uint32_t t, float* 
     }
 }
 
-// A workgroup takes `tile` consecutive rows; with a convolution it also stages the taps - 1 rows in front of them (from its own
+// The general form (any width and number of taps the LDS holds).  A workgroup takes `tile` consecutive rows; with a convolution it also stages the taps - 1 rows in front of them (from its own
 // inputs, or from the ring for positions before this portion).  Only the first workgroup reads the ring (tile >= taps - 1), and it
 // alone writes it, after its reads: the last rows of the portion, recomputed.
 template <int MODE, bool CONV, typename AT>
@@ -67,7 +78,7 @@ __global__ __launch_bounds__(256) void rows_kernel(RowsArgs a, uint32_t tile) {
         float* h = hrow + (size_t)r * dim;
         if (j < 0) {
             const int p = (int)a.pos0 + j;
-            const float* past = p >= 0 ? s.ring + (size_t)((uint32_t)p % s.taps) * dim : nullptr;
+            const float* past = p >= 0 ? s.ring + (size_t)((uint32_t)p % s.taps) * s.x_stride : nullptr;
             for (uint32_t e = lane; e < dim; e += 64) h[e] = past ? past[e] : 0.0f;
             continue;
         }
@@ -92,7 +103,7 @@ __global__ __launch_bounds__(256) void rows_kernel(RowsArgs a, uint32_t tile) {
                 if constexpr (CONV) {
                     const float h = v;
                     float c = 0.0f;
-                    for (uint32_t k = 0; k < s.taps; k++) c += s.conv[(size_t)k * dim + e] * hrow[(size_t)(r + k) * dim + e];
+                    for (uint32_t k = 0; k < s.taps; k++) c += s.conv[(size_t)k * s.x_stride + e] * hrow[(size_t)(r + k) * dim + e];
                     v = h + c;
                 }
             }
@@ -107,7 +118,167 @@ __global__ __launch_bounds__(256) void rows_kernel(RowsArgs a, uint32_t tile) {
     }
     if (CONV && blockIdx.x == 0) {
         const uint32_t first = a.n > s.taps ? a.n - s.taps : 0u;
-        for (uint32_t j = first + wave; j < a.n; j += 4) stage_row<true>(s, j, s.ring + (size_t)((a.pos0 + j) % s.taps) * dim, nullptr);
+        for (uint32_t j = first + wave; j < a.n; j += 4) stage_row<true>(s, j, s.ring + (size_t)((a.pos0 + j) % s.taps) * s.x_stride, nullptr);
+    }
+}
+
+// ---- the fast form: up to four taps, up to 4096 coordinates -------------------------------------------------------------------
+// A thread owns four neighbouring coordinates of R consecutive rows and keeps them in registers: all loads of the tile are in flight
+// together, the R sums of squares go through one exchange, and the convolution, which runs along the rows, never leaves the thread.
+constexpr int kHalo = 3;
+
+__device__ __forceinline__ v4f load4(const float* p) { return *reinterpret_cast<const v4f*>(p); }
+__device__ __forceinline__ v4f mask4(v4f v, uint32_t e, uint32_t dim) {
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+        if (e + i >= dim) v[i] = 0.0f;
+    return v;
+}
+__device__ __forceinline__ float dot4(v4f a, v4f b) { return (a[0] * b[0] + a[1] * b[1]) + (a[2] * b[2] + a[3] * b[3]); }
+
+// sum[r] over the workgroup for R values per thread.  red: [R][NT / 64].
+template <int R, int NT>
+__device__ __forceinline__ void block_sums(float (&v)[R], float* red) {
+    constexpr int W = NT / 64;
+    __syncthreads();  // red may still be read from an earlier call
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const float w = wave_sum_f32(v[r]);
+        if ((threadIdx.x & 63u) == 0) red[r * W + (threadIdx.x >> 6)] = w;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        float t = 0.0f;
+#pragma unroll
+        for (int w = 0; w < W; w++) t += red[r * W + w];
+        v[r] = t;
+    }
+}
+
+// Rows first .. first + R - 1 (clamped to n - 1; negative ones are left at zero): h[r] = x + g_post y / rms(y), normed when NORM;
+// rows from `own` on are stored to x_out.
+template <bool NORM, int R, int NT>
+__device__ __forceinline__ void stage_tile(const RowsArgs& a, int first, int own, v4f (&h)[R], float* red) {
+    const RowStage& s = a.s;
+    const uint32_t e = 4u * threadIdx.x;
+    const bool on = e < s.dim, has_y = s.y || s.experts;
+    v4f y[R];
+    uint32_t row[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const int j = first + r < (int)a.n ? first + r : (int)a.n - 1;
+        row[r] = j < 0 ? 0u : a.rows ? a.rows[j] : (uint32_t)j;
+        h[r] = y[r] = v4f{0.f, 0.f, 0.f, 0.f};
+        if (!on || first + r < 0) continue;
+        h[r] = load4(s.x + (size_t)row[r] * s.x_stride + e);
+        if (s.y) y[r] = load4(s.y + (size_t)row[r] * s.y_stride + e);
+    }
+    if (s.experts) {
+        const float share = 1.0f / (float)s.top;
+        for (uint32_t k = 0; k < s.top; k++) {
+            v4f v[R];
+#pragma unroll
+            for (int r = 0; r < R; r++)
+                v[r] = on && first + r >= 0 ? load4(s.experts + (size_t)s.slots[(size_t)row[r] * s.top + k] * s.y_stride + e) : v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int r = 0; r < R; r++) y[r] += v[r] * share;
+        }
+    }
+    float ss[R];
+    if (has_y) {
+#pragma unroll
+        for (int r = 0; r < R; r++) y[r] = mask4(y[r], e, s.dim), ss[r] = dot4(y[r], y[r]);
+        block_sums<R, NT>(ss, red);
+#pragma unroll
+        for (int r = 0; r < R; r++) h[r] += y[r] * (s.g_post / sqrtf(ss[r] / (float)s.dim + s.eps));
+    }
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        h[r] = mask4(h[r], e, s.dim);
+        if (s.x_out && on && r >= own && first + r < (int)a.n) *reinterpret_cast<v4f*>(s.x_out + (size_t)row[r] * s.x_stride + e) = h[r];
+    }
+    if constexpr (NORM) {
+#pragma unroll
+        for (int r = 0; r < R; r++) ss[r] = dot4(h[r], h[r]);
+        block_sums<R, NT>(ss, red);
+#pragma unroll
+        for (int r = 0; r < R; r++) h[r] *= s.g_pre / sqrtf(ss[r] / (float)s.dim + s.eps);
+    }
+}
+
+template <int MODE, bool CONV, int R, int NT, typename AT>
+__global__ __launch_bounds__(NT) void rows_fast_kernel(RowsArgs a) {
+    constexpr int HALO = CONV ? kHalo : 0, TILE = R - HALO;
+    __shared__ float red[R * (NT / 64)];
+    const RowStage& s = a.s;
+    const uint32_t e = 4u * threadIdx.x;
+    const int j0 = (int)blockIdx.x * TILE;
+    v4f w[kHalo + 1], h[R];
+    if constexpr (CONV) {
+#pragma unroll
+        for (int m = 0; m <= kHalo; m++)  // by distance: the newest input is the last tap
+            w[m] = m < (int)s.taps && e < s.dim ? mask4(load4(s.conv + (size_t)(s.taps - 1u - m) * s.x_stride + e), e, s.dim) : v4f{0.f, 0.f, 0.f, 0.f};
+    }
+    stage_tile<MODE == kRowNorm, R, NT>(a, j0 - HALO, HALO, h, red);
+    if constexpr (MODE == kRowOnly) return;
+    if constexpr (CONV) {
+        if (j0 == 0) {  // the inputs in front of this portion
+#pragma unroll
+            for (int r = 0; r < HALO; r++) {
+                const int p = (int)a.pos0 + r - HALO;
+                h[r] = p >= 0 && HALO - r < (int)s.taps && e < s.dim ? mask4(load4(s.ring + (size_t)((uint32_t)p % s.taps) * s.x_stride + e), e, s.dim)
+                                                                      : v4f{0.f, 0.f, 0.f, 0.f};
+            }
+        }
+    }
+    if (MODE == kRowNorm && !CONV && a.gate_w) {
+        float d[R];
+        const uint2 g = e < a.kp ? *reinterpret_cast<const uint2*>(a.gate_w + e) : uint2{0, 0};
+        const v4f gw = {__uint_as_float(g.x << 16), __uint_as_float(g.x & 0xffff0000u), __uint_as_float(g.y << 16), __uint_as_float(g.y & 0xffff0000u)};
+#pragma unroll
+        for (int r = 0; r < R; r++) d[r] = dot4(h[r], gw);
+        block_sums<R, NT>(d, red);
+        if (threadIdx.x == 0) {
+#pragma unroll
+            for (int r = 0; r < R; r++)
+                if (j0 + r < (int)a.n) a.row_gate[j0 + r] = 1.0f / (1.0f + expf(-d[r]));
+        }
+    }
+#pragma unroll
+    for (int r = HALO; r < R; r++) {
+        const int j = j0 + r - HALO;
+        if (j >= (int)a.n || e >= a.kp) continue;
+        v4f v = h[r];
+        if constexpr (CONV) {
+            v4f c = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int m = kHalo; m >= 0; m--) c += w[m] * h[r - m];
+            v += c;
+        }
+        AT* o = static_cast<AT*>(a.out) + (size_t)j * a.ldo + e;
+        if constexpr (MODE == kRowSplit && sizeof(AT) == 2) {
+            v4f hi;
+#pragma unroll
+            for (int i = 0; i < 4; i++) hi[i] = (float)(__bf16)v[i];
+            store4(o, hi), store4(o + a.lo_at, v - hi);
+        } else {
+            store4(o, v);
+        }
+    }
+    if constexpr (CONV) {
+        if (j0 == 0) {  // the only workgroup that reads the ring writes it: the portion's last inputs
+            v4f tail[kHalo + 1];
+            RowsArgs b = a;
+            b.s.x_out = nullptr;
+            stage_tile<true, kHalo + 1, NT>(b, (int)a.n - kHalo - 1, kHalo + 1, tail, red);
+#pragma unroll
+            for (int r = 0; r <= kHalo; r++) {
+                const int j = (int)a.n - kHalo - 1 + r;
+                if (j >= 0 && kHalo + 1 - r <= (int)s.taps && e < s.dim)
+                    *reinterpret_cast<v4f*>(s.ring + (size_t)((a.pos0 + (uint32_t)j) % s.taps) * s.x_stride + e) = tail[r];
+            }
+        }
     }
 }
 
@@ -142,7 +313,7 @@ __global__ __launch_bounds__(256) void route_kernel(const RouteJob* __restrict__
     __syncthreads();
     if (tid == 0) {
         uint32_t se = 0, st = 0;
-        for (uint32_t i = 0; i < 256; i++) {
+        for (uint32_t i = 0; i < (job.experts + per - 1u) / per; i++) {
             const uint32_t ce = chunk_entries[i], ct = chunk_tiles[i];
             chunk_entries[i] = se, chunk_tiles[i] = st;
             se += ce, st += ct;
@@ -169,6 +340,17 @@ __global__ __launch_bounds__(256) void route_kernel(const RouteJob* __restrict__
 
 template <int MODE, bool CONV, typename AT>
 hipError_t run_rows(const RowsArgs& a, const Launch& L) {
+    const uint32_t kp = MODE == kRowOnly ? a.s.dim : a.kp;
+    const bool aligned = a.s.x_stride % 4u == 0 && (a.s.y_stride % 4u == 0) && a.ldo % 4u == 0 && a.lo_at % 4u == 0 && kp <= pad_to(a.s.dim, kDensePad) &&
+                         pad_to(a.s.dim, kDensePad) <= a.s.x_stride && (!(a.s.y || a.s.experts) || pad_to(a.s.dim, kDensePad) <= a.s.y_stride);
+    if (aligned && kp <= 4096u && (!CONV || a.s.taps <= (uint32_t)kHalo + 1u)) {
+        constexpr int R = CONV ? 11 : 4;
+        const dim3 grid((a.n + R - (CONV ? kHalo : 0) - 1) / (R - (CONV ? kHalo : 0)));
+        if (kp <= 1024u) return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, R, 256, AT>, grid, dim3(256), a);
+        if (kp <= 2048u) return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, R, 512, AT>, grid, dim3(512), a);
+        return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, CONV ? 7 : 4, 1024, AT>,
+                             CONV ? dim3((a.n + 3u) / 4u) : grid, dim3(1024), a);
+    }
     const uint32_t halo = CONV ? a.s.taps - 1u : 0u;
     uint32_t tile = 8;
     while (tile > 1 && tile / 2 >= halo && (size_t)(tile + halo) * a.s.dim * 4u > 64u * 1024u) tile /= 2;

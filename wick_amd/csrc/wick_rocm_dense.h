@@ -34,8 +34,8 @@ struct RowStage {
     float g_post = 0.0f, g_pre = 0.0f, eps = 0.0f;
     uint32_t dim = 0;
     float* x_out = nullptr;        // [n][x_stride], never aliases x; null: not kept
-    const float* conv = nullptr;   // [taps][dim]; null: no convolution
-    float* ring = nullptr;         // [taps][dim]
+    const float* conv = nullptr;   // [taps][x_stride]; null: no convolution
+    float* ring = nullptr;         // [taps][x_stride]
     uint32_t taps = 0;
     // y as the weighted outputs of routed experts: y += (1 / top) * sum_s experts[slot(t, s)] (prompt passes only)
     const float* experts = nullptr;     // [n * top][y_stride]
