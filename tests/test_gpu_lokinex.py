@@ -92,6 +92,11 @@ ONE = {
     "moe_many": S.config([S.layer(S.latent(), S.moe(ff=16, experts=300, top=4, shared=8))], vocab=400),
     "loop_all": S.config([S.layer(S.rglru(), S.dense())], loop=(0, 1, 3)),
     "loop_once": S.config([S.layer(S.rglru()), S.layer(S.latent())], loop=(1, 2, 1)),
+    "long_convolutions": S.config([S.layer(S.rglru(width=48, blocks=2, conv=7), S.dense(32)), S.layer(S.latent())], width=72, taps=6),
+    "long_and_wide": S.config([S.layer(S.rglru(width=64, blocks=1, conv=8))], width=1500, taps=6, vocab=60),
+    "width_2000": S.config([S.layer(S.rglru(width=64, blocks=1), S.moe(ff=24)), S.layer(S.latent(), S.dense(96))], width=2000, vocab=60),
+    "width_3000": S.config([S.layer(S.rglru(width=64, blocks=1), S.moe(ff=24))], width=3000, vocab=60, loop=(0, 1, 2)),
+    "width_4200": S.config([S.layer(S.rglru(width=64, blocks=1), S.dense(24))], width=4200, vocab=60, loop=(0, 1, 2)),
     "odd_width": S.config([S.layer(S.rglru(width=33, blocks=3, conv=3), S.dense(7)), S.layer(S.latent(), S.moe(ff=5, shared=3))], width=101, vocab=37, taps=3),
     "mixed": S.mixed(),
     "mixed_loop_to_the_end": S.mixed(loop=(2, 4, 2)),
@@ -279,6 +284,15 @@ def test_large_products_and_several_passes(ctx, tmp_path):
         served.restore_state(state, 2150)
         assert np.array_equal(served.forward([3], 2150), step)
         assert error(exact.forward(toks[:150], 0, [149]), first[-1]) <= TOL_F32
+
+
+@BOTH
+def test_portions_with_long_convolutions(ctx, tmp_path, dtype):
+    with Pair(ctx, tmp_path, ONE["long_convolutions"], dtype, seed=15) as p:
+        toks = p.tokens(60, 1)
+        want = p.want(toks)
+        for cuts in ([60], [3] * 20, [4, 2, 1, 3, 5, 6, 7, 32], [1, 59]):
+            p.check(p.portions(toks, cuts), want)
 
 
 @BOTH

@@ -4,7 +4,8 @@
 // Two bodies share the epilogues, because the 16 x 16 result of v_mfma_f32_16x16x32_bf16 and of v_mfma_f32_16x16x4_f32 sits in the
 // same registers (lane l: column l % 16, rows 4 (l / 16) + r):
 //   gemm_bf16_kernel  activations in bfloat16; 2 x 2 waves of (16 MT) x (16 NT) outputs, K in steps of 64 through two LDS buffers
-//                     (the next step's global loads are in flight during the products of this one); the 16-byte chunks of an LDS
+//                     (the global loads of the next PD steps are in flight during the products of this one: a tile of a small
+//                     product is alone on its CU, and a step's products are much shorter than a trip to memory); the 16-byte chunks of an LDS
 //                     row are permuted by row % 8, so that the 16 rows a fragment read touches spread over the banks;
 //   gemm_f32_kernel   activations in f32, weights widened exactly: every product and sum in f32.
 // Weights are the M side, so a lane ends with four consecutive features of one token: one vector store.  With TRANS the sides are
@@ -197,7 +198,7 @@ __device__ __forceinline__ void run_epilogue(const GemmArgs& a, const TileAt& o,
     }
 }
 
-template <int MT, int NT, class Epi>
+template <int MT, int NT, int PD, class Epi>
 __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
     constexpr uint32_t BM = 32 * MT, BN = 32 * NT, BK = 64;
     constexpr int LA = BM * 8 / 256, LB = BN * 8 / 256;  // 16-byte chunks per thread and step
@@ -221,52 +222,60 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
         pb[i] = x + (size_t)source_row(a, o, row) * a.ldx + ch * 8;
         db[i] = row * BK + ((ch ^ (row & 7u)) << 3);
     }
-    u4 ra[LA], rb[LB];
+    const uint32_t steps = a.k / BK;
+    u4 ra[PD][LA], rb[PD][LB];
 #pragma unroll
-    for (int i = 0; i < LA; i++) ra[i] = *reinterpret_cast<const u4*>(pa[i]);
+    for (int d = 0; d < PD; d++) {
+        const uint32_t k0 = (uint32_t)d < steps ? BK * d : 0u;
 #pragma unroll
-    for (int i = 0; i < LB; i++) rb[i] = *reinterpret_cast<const u4*>(pb[i]);
+        for (int i = 0; i < LA; i++) ra[d][i] = *reinterpret_cast<const u4*>(pa[i] + k0);
+#pragma unroll
+        for (int i = 0; i < LB; i++) rb[d][i] = *reinterpret_cast<const u4*>(pb[i] + k0);
+    }
     v4f acc[MT][NT];
 #pragma unroll
     for (int i = 0; i < MT; i++)
 #pragma unroll
         for (int j = 0; j < NT; j++) acc[i][j] = v4f{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int i = 0; i < LA; i++) *reinterpret_cast<u4*>(&sa[0][da[i]]) = ra[i];
-#pragma unroll
-    for (int i = 0; i < LB; i++) *reinterpret_cast<u4*>(&sb[0][db[i]]) = rb[i];
-    __syncthreads();
+    // Step s + 1 leaves its registers for LDS behind the products of step s, and step s + 1 + PD is requested into them.
     int cur = 0;
-    for (uint32_t k0 = 0; k0 < a.k; k0 += BK, cur ^= 1) {
-        const bool more = k0 + BK < a.k;
-        if (more) {
+    auto advance = [&](u4 (&va)[LA], u4 (&vb)[LB], uint32_t refill, int buf) {
 #pragma unroll
-            for (int i = 0; i < LA; i++) ra[i] = *reinterpret_cast<const u4*>(pa[i] + k0 + BK);
+        for (int i = 0; i < LA; i++) *reinterpret_cast<u4*>(&sa[buf][da[i]]) = va[i];
 #pragma unroll
-            for (int i = 0; i < LB; i++) rb[i] = *reinterpret_cast<const u4*>(pb[i] + k0 + BK);
+        for (int i = 0; i < LB; i++) *reinterpret_cast<u4*>(&sb[buf][db[i]]) = vb[i];
+        if (refill >= steps) return;
+#pragma unroll
+        for (int i = 0; i < LA; i++) va[i] = *reinterpret_cast<const u4*>(pa[i] + refill * BK);
+#pragma unroll
+        for (int i = 0; i < LB; i++) vb[i] = *reinterpret_cast<const u4*>(pb[i] + refill * BK);
+    };
+    advance(ra[0], rb[0], PD, 0);
+    __syncthreads();
+    for (uint32_t s0 = 0; s0 < steps; s0 += PD) {
+#pragma unroll
+        for (int d = 0; d < PD; d++) {
+            const uint32_t step = s0 + d;
+            if (step >= steps) break;
+#pragma unroll
+            for (int s = 0; s < 2; s++) {
+                bf8 fa[MT], fb[NT];
+                const uint32_t ch = (((4 * s + g) ^ (l16 & 7u)) << 3);
+#pragma unroll
+                for (int i = 0; i < MT; i++) fa[i] = *reinterpret_cast<const bf8*>(&sa[cur][(wm + 16 * i + l16) * BK + ch]);
+#pragma unroll
+                for (int j = 0; j < NT; j++) fb[j] = *reinterpret_cast<const bf8*>(&sb[cur][(wn + 16 * j + l16) * BK + ch]);
+#pragma unroll
+                for (int i = 0; i < MT; i++)
+#pragma unroll
+                    for (int j = 0; j < NT; j++)
+                        acc[i][j] = Epi::kTrans ? __builtin_amdgcn_mfma_f32_16x16x32_bf16(fb[j], fa[i], acc[i][j], 0, 0, 0)
+                                                : __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+            }
+            if (step + 1 < steps) advance(ra[(d + 1) % PD], rb[(d + 1) % PD], step + 1 + PD, cur ^ 1);
+            __syncthreads();
+            cur ^= 1;
         }
-#pragma unroll
-        for (int s = 0; s < 2; s++) {
-            bf8 fa[MT], fb[NT];
-            const uint32_t ch = (((4 * s + g) ^ (l16 & 7u)) << 3);
-#pragma unroll
-            for (int i = 0; i < MT; i++) fa[i] = *reinterpret_cast<const bf8*>(&sa[cur][(wm + 16 * i + l16) * BK + ch]);
-#pragma unroll
-            for (int j = 0; j < NT; j++) fb[j] = *reinterpret_cast<const bf8*>(&sb[cur][(wn + 16 * j + l16) * BK + ch]);
-#pragma unroll
-            for (int i = 0; i < MT; i++)
-#pragma unroll
-                for (int j = 0; j < NT; j++)
-                    acc[i][j] = Epi::kTrans ? __builtin_amdgcn_mfma_f32_16x16x32_bf16(fb[j], fa[i], acc[i][j], 0, 0, 0)
-                                            : __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
-        }
-        if (more) {
-#pragma unroll
-            for (int i = 0; i < LA; i++) *reinterpret_cast<u4*>(&sa[cur ^ 1][da[i]]) = ra[i];
-#pragma unroll
-            for (int i = 0; i < LB; i++) *reinterpret_cast<u4*>(&sb[cur ^ 1][db[i]]) = rb[i];
-        }
-        __syncthreads();
     }
     run_epilogue<MT, NT>(a, o, epi, acc, wm, wn, l16, g);
 }
@@ -334,12 +343,12 @@ hipError_t run_gemm(const DenseWeight& w, const GemmIn& in, const Epi& epi, cons
         return dim3(mt * nt, 1, z);
     };
     if (in.f32) return launch_kernel(L, kFamGemm, gemm_f32_kernel<Epi>, grid(64, 64), dim3(256), a, epi);
-    if (g.tiles) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, Epi>, grid(128, kGroupTileRows), dim3(256), a, epi);
+    if (g.tiles) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, 3, Epi>, grid(128, kGroupTileRows), dim3(256), a, epi);
     // the widest tile that leaves no CU without one (a short K is mostly epilogue: small tiles, more of them)
     const dim3 big = grid(128, 128), tall = grid(128, 64);
-    if (w.kp > 256u && big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, Epi>, big, dim3(256), a, epi);
-    if (w.kp > 256u && tall.x * tall.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, Epi>, tall, dim3(256), a, epi);
-    return launch_kernel(L, kFamGemm, gemm_bf16_kernel<2, 2, Epi>, grid(64, 64), dim3(256), a, epi);
+    if (w.kp > 256u && big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, 2, Epi>, big, dim3(256), a, epi);
+    if (w.kp > 256u && tall.x * tall.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, 3, Epi>, tall, dim3(256), a, epi);
+    return launch_kernel(L, kFamGemm, gemm_bf16_kernel<2, 2, 4, Epi>, grid(64, 64), dim3(256), a, epi);
 }
 
 }  // namespace

@@ -21,7 +21,7 @@ typedef uint32_t u4 __attribute__((ext_vector_type(4)));
 constexpr uint32_t kChunk = 64;      // positions per pass
 constexpr uint32_t kMaxSplits = 64;  // workgroups along the sequence
 constexpr uint32_t kSlab = 128;      // latent columns per workgroup of the absorbing launch
-constexpr uint32_t kStageBytes = 144u * 1024u;  // dynamic LDS of the staged form, beside its static 6 KB
+constexpr uint32_t kStageBytes = 136u * 1024u;  // dynamic LDS of the staged form, beside at most 21 KB of its own
 constexpr float kLog2e = 1.44269504088896340736f;
 
 __device__ __forceinline__ void put(float* p, float v) { *p = v; }
@@ -172,7 +172,7 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
     extern __shared__ __align__(16) float qs[];  // [HG][row], then STAGED: [kChunk][row] of the cache type
     __shared__ __align__(16) float sc[HG][kChunk], wt[kChunk][HG];
     __shared__ float corr[HG];
-    __shared__ float red[256 * 2];
+    __shared__ float2 red[HG][256];
     const LatentShape& s = a.s;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, row = s.row();
     const uint32_t split = blockIdx.x, h0 = blockIdx.y * HG, t = blockIdx.z;
@@ -180,6 +180,14 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
     if (pos >= s.max_seq || split * kChunk > pos) return;  // the merge derives the number of partials from pos as well
     const CT* cache = static_cast<const CT*>(a.cache);
     const uint32_t nh = s.heads - h0 < (uint32_t)HG ? s.heads - h0 : (uint32_t)HG;
+    constexpr uint32_t PER = 16 / sizeof(CT), AHEAD = 12;  // elements of a 16-byte piece; pieces a thread has in flight
+    u4 ahead[STAGED ? AHEAD : 1];
+    auto fetch = [&](const CT* rows, uint32_t pieces, uint32_t i0) {
+#pragma unroll
+        for (uint32_t j = 0; j < (STAGED ? AHEAD : 1u); j++) ahead[j] = *reinterpret_cast<const u4*>(rows + (size_t)(i0 + 256u * j < pieces ? i0 + 256u * j : 0u) * PER);
+    };
+    auto chunk_keys = [&](uint32_t c) { return pos + 1u - c * kChunk < kChunk ? pos + 1u - c * kChunk : kChunk; };
+    if constexpr (STAGED) fetch(cache + (size_t)split * kChunk * row, chunk_keys(split) * (row / PER), tid);  // ... before the queries
     for (uint32_t i = tid; i < HG * row; i += 256) {
         const uint32_t h = i / row;
         qs[i] = a.qa[((size_t)t * s.heads + h0 + (h < nh ? h : 0u)) * row + i % row];  // absent heads repeat the first one
@@ -199,19 +207,16 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
     const uint32_t l16 = lane & 15u, key_in = wave * 16u + (lane >> 4) * 4u;  // this lane group's four positions of a chunk
 
     for (uint32_t c = split; c * kChunk <= pos; c += a.splits) {
-        const uint32_t t0 = c * kChunk, nt = pos + 1u - t0 < kChunk ? pos + 1u - t0 : kChunk;
+        const uint32_t t0 = c * kChunk, nt = chunk_keys(c);
         const CT* rows = cache + (size_t)t0 * row;
         if constexpr (STAGED) {
-            constexpr uint32_t PER = 16 / sizeof(CT);
             CT* stage = reinterpret_cast<CT*>(qs + HG * row);
             const uint32_t pieces = nt * (row / PER);
-            for (uint32_t i0 = tid; i0 < pieces; i0 += 8u * 256u) {
-                u4 v[8];
+            for (uint32_t i0 = tid; i0 < pieces; i0 += AHEAD * 256u) {
+                if (c != split || i0 != tid) fetch(rows, pieces, i0);
 #pragma unroll
-                for (int j = 0; j < 8; j++) v[j] = *reinterpret_cast<const u4*>(rows + (size_t)(i0 + 256u * j < pieces ? i0 + 256u * j : i0) * PER);
-#pragma unroll
-                for (int j = 0; j < 8; j++)
-                    if (i0 + 256u * j < pieces) *reinterpret_cast<u4*>(stage + (size_t)(i0 + 256u * j) * PER) = v[j];
+                for (uint32_t j = 0; j < AHEAD; j++)
+                    if (i0 + 256u * j < pieces) *reinterpret_cast<u4*>(stage + (size_t)(i0 + 256u * j) * PER) = ahead[j];
             }
             rows = stage;
             __syncthreads();
@@ -292,22 +297,23 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
         }
         __syncthreads();  // sc, wt and corr are rewritten by the next chunk
     }
+    auto part_of = [&](int h) { return a.part + (((size_t)t * s.heads + h0 + h) * a.splits + split) * (s.rank_p + 4u); };
 #pragma unroll
-    for (int h = 0; h < HG; h++) {
-        float* part = a.part + (((size_t)t * s.heads + h0 + h) * a.splits + split) * (s.rank_p + 4u);
-        const bool live = h < (int)nh;
-        if (live && wave == (uint32_t)(h & 3) && lane == 0) part[0] = m_run[h >> 2], part[1] = l_run[h >> 2];
+    for (int h = 0; h < HG; h++)
+        if (h < (int)nh && wave == (uint32_t)(h & 3) && lane == 0) part_of(h)[0] = m_run[h >> 2], part_of(h)[1] = l_run[h >> 2];
 #pragma unroll
-        for (int i = 0; i < NP; i++) {
-            __syncthreads();
-            red[2 * tid] = acc[i][h][0], red[2 * tid + 1] = acc[i][h][1];
-            __syncthreads();
-            const uint32_t p = cp + 256u * i;
-            if (live && kg == 0 && p < pairs) {
-                float v0 = 0.0f, v1 = 0.0f;
-                for (uint32_t g = 0; g < kgroups; g++) v0 += red[2 * (g * cpp + cp)], v1 += red[2 * (g * cpp + cp) + 1];
-                part[4 + 2 * p] = v0, part[4 + 2 * p + 1] = v1;
-            }
+    for (int i = 0; i < NP; i++) {
+        if (i > 0) __syncthreads();
+#pragma unroll
+        for (int h = 0; h < HG; h++) red[h][tid] = float2{acc[i][h][0], acc[i][h][1]};
+        __syncthreads();
+        for (uint32_t x = tid; x < HG * cpp; x += 256u) {
+            const uint32_t h = x / cpp, p = x % cpp + 256u * i;
+            if (h >= nh || p >= pairs) continue;
+            float2 v = {0.0f, 0.0f};
+            for (uint32_t g = 0; g < kgroups; g++) v.x += red[h][g * cpp + x % cpp].x, v.y += red[h][g * cpp + x % cpp].y;
+            float* part = part_of((int)h) + 4 + 2 * p;
+            part[0] = v.x, part[1] = v.y;
         }
     }
 }
@@ -327,6 +333,7 @@ template <typename OT>
 __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
     extern __shared__ __align__(16) float oc[];  // [rank_p]
     __shared__ float wts[kMaxSplits];
+    __shared__ v4f sums[256];
     const LatentShape& s = a.s;
     const uint32_t h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x, lane = tid & 63u;
     const uint32_t pos = (a.d_pos ? *a.d_pos : a.pos0) + t;
@@ -343,6 +350,20 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
     active = active < a.splits ? active : a.splits;
     const uint32_t stride = s.rank_p + 4u;
     const float* parts = a.part + ((size_t)t * s.heads + h) * a.splits * stride;
+    // thread (group of partials, four latent columns)
+    const uint32_t quads = s.rank_p / 4u;
+    uint32_t cols = 8;
+    while (cols < 256u && cols < quads) cols <<= 1;
+    const uint32_t groups = 256u / cols, grp = tid / cols;
+    v4f pre[8];
+    auto fetch = [&](uint32_t quad, uint32_t i0) {
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+            const uint32_t i = i0 + j * groups;
+            pre[j] = quad < quads ? *reinterpret_cast<const v4f*>(parts + (size_t)(i < active ? i : 0u) * stride + 4 + 4 * quad) : v4f{0.f, 0.f, 0.f, 0.f};
+        }
+    };
+    fetch(tid % cols, grp);
     if (tid < 64) {
         const bool on = tid < active;
         const float m_i = on ? parts[(size_t)tid * stride] : -__builtin_inff(), l_i = on ? parts[(size_t)tid * stride + 1] : 0.0f;
@@ -350,16 +371,25 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
         wts[tid] = w / l;
     }
     __syncthreads();
-    for (uint32_t e = tid; e < s.rank_p; e += 256) {
-        float v = 0.0f;
-        for (uint32_t i0 = 0; i0 < active; i0 += 8) {
-            float p[8];
+    for (uint32_t quad = tid % cols; quad < quads || quad == tid % cols; quad += cols) {
+        v4f v = {0.f, 0.f, 0.f, 0.f};
+        for (uint32_t i0 = grp; i0 < active; i0 += 8u * groups) {
+            if (quad != tid % cols || i0 != grp) fetch(quad, i0);
 #pragma unroll
-            for (int j = 0; j < 8; j++) p[j] = parts[(size_t)(i0 + j < active ? i0 + j : i0) * stride + 4 + e];
-#pragma unroll
-            for (int j = 0; j < 8; j++) v += i0 + j < active ? p[j] * wts[i0 + j] : 0.0f;
+            for (int j = 0; j < 8; j++) {
+                const uint32_t i = i0 + j * groups;
+                if (i < active) v += pre[j] * wts[i];
+            }
         }
-        oc[e] = v;
+        if (groups > 1) {  // then one quad per thread (cols >= quads)
+            sums[tid] = v;
+            __syncthreads();
+            if (grp == 0) {
+                v = sums[tid];
+                for (uint32_t g = 1; g < groups; g++) v += sums[g * cols + tid];
+            }
+        }
+        if (grp == 0 && quad < quads) *reinterpret_cast<v4f*>(oc + 4 * quad) = v;
     }
     __syncthreads();
     OT* out = static_cast<OT*>(a.out) + (size_t)t * a.ldo;
@@ -604,7 +634,9 @@ hipError_t launch_latent_attention(const LatentShape& s, const LatentWeights& w,
         return attend(hg, std::integral_constant<int, 4>{});
     };
     // LDS holds the queries of a group of heads: eight while they leave room for a second workgroup
-    hipError_t e = n > 1 && s.row() <= 1024u ? with_pairs(std::integral_constant<int, 8>{}) : with_pairs(std::integral_constant<int, 4>{});
+    hipError_t e = n == 1 && s.heads <= 16u ? with_pairs(std::integral_constant<int, 2>{})  // one token: more workgroups with less to do
+                   : n > 1 && s.row() <= 1024u ? with_pairs(std::integral_constant<int, 8>{})
+                                                : with_pairs(std::integral_constant<int, 4>{});
     if (e != hipSuccess) return e;
     const MergeArgs m{s, scratch, pos0, splits, d_pos, w.uv, out, ldo, kp};
     const dim3 grid(s.heads, n, n == 1 ? 4 : 1);
