@@ -1,4 +1,5 @@
-"""Plain, slow numpy implementation of the Lokinex design: the checker of the GPU model (test infrastructure only).
+"""Plain, slow numpy implementation of the Lokinex design: what the GPU model is compared with (test infrastructure
+only).
 
 One function per mechanism, each over a whole sequence [T, ...] with an explicit state for what came before it, everything in
 float64 unless a test asks for another type.  No code is shared with the product path.

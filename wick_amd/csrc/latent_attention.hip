@@ -87,7 +87,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(AbsorbArgs a) {
     v4f acc = {0.f, 0.f, 0.f, 0.f};
     if (col < s.rank_p) {
         const uint16_t* w = a.w.uk + (size_t)h * s.dim * s.rank_p + col;
-#pragma unroll 4
+#pragma unroll 8
         for (uint32_t d = grp; d < s.dim; d += 8) {
             const uint2 k = *reinterpret_cast<const uint2*>(w + (size_t)d * s.rank_p);
             const float qv = q[d];
@@ -176,10 +176,13 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
     const LatentShape& s = a.s;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, row = s.row();
     const uint32_t split = blockIdx.x, h0 = blockIdx.y * HG, t = blockIdx.z;
+    const uint32_t nh = s.heads - h0 < (uint32_t)HG ? s.heads - h0 : (uint32_t)HG;
+    const float* qa = a.qa + ((size_t)t * s.heads + h0) * row;  // rows of a token's heads follow each other
+    const uint32_t q_len = nh * row;
+    const v4f q_first = 4u * tid < q_len ? *reinterpret_cast<const v4f*>(qa + 4u * tid) : v4f{0.f, 0.f, 0.f, 0.f};
     const uint32_t pos = (a.d_pos ? *a.d_pos : a.pos0) + t;
     if (pos >= s.max_seq || split * kChunk > pos) return;  // the merge derives the number of partials from pos as well
     const CT* cache = static_cast<const CT*>(a.cache);
-    const uint32_t nh = s.heads - h0 < (uint32_t)HG ? s.heads - h0 : (uint32_t)HG;
     constexpr uint32_t PER = 16 / sizeof(CT), AHEAD = 12;  // elements of a 16-byte piece; pieces a thread has in flight
     u4 ahead[STAGED ? AHEAD : 1];
     auto fetch = [&](const CT* rows, uint32_t pieces, uint32_t i0) {
@@ -188,9 +191,9 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(AttendArgs a) {
     };
     auto chunk_keys = [&](uint32_t c) { return pos + 1u - c * kChunk < kChunk ? pos + 1u - c * kChunk : kChunk; };
     if constexpr (STAGED) fetch(cache + (size_t)split * kChunk * row, chunk_keys(split) * (row / PER), tid);  // ... before the queries
-    for (uint32_t i = tid; i < HG * row; i += 256) {
-        const uint32_t h = i / row;
-        qs[i] = a.qa[((size_t)t * s.heads + h0 + (h < nh ? h : 0u)) * row + i % row];  // absent heads repeat the first one
+    for (uint32_t i = 4u * tid; i < HG * row; i += 1024u) {  // absent heads: zeros
+        const v4f q = i == 4u * tid ? q_first : i < q_len ? *reinterpret_cast<const v4f*>(qa + i) : v4f{0.f, 0.f, 0.f, 0.f};
+        *reinterpret_cast<v4f*>(qs + i) = q;
     }
     __syncthreads();
     const uint32_t pairs = s.rank_p / 2u;
@@ -336,8 +339,6 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
     __shared__ v4f sums[256];
     const LatentShape& s = a.s;
     const uint32_t h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x, lane = tid & 63u;
-    const uint32_t pos = (a.d_pos ? *a.d_pos : a.pos0) + t;
-    if (pos >= s.max_seq) return;
     // the first four value rows of a wave are requested before the partials are looked at (rank_p <= 512: whole rows)
     const uint32_t waves = gridDim.z * 4u, first = blockIdx.z * 4u + (tid >> 6);
     float ahead[4][8];
@@ -346,8 +347,6 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
         const uint32_t v = first + r * waves < s.vdim ? first + r * waves : s.vdim - 1u;
         if (8u * lane < s.rank_p) load8(a.uv + ((size_t)h * s.vdim + v) * s.rank_p + 8u * lane, ahead[r]);
     }
-    uint32_t active = pos / kChunk + 1u;
-    active = active < a.splits ? active : a.splits;
     const uint32_t stride = s.rank_p + 4u;
     const float* parts = a.part + ((size_t)t * s.heads + h) * a.splits * stride;
     // thread (group of partials, four latent columns)
@@ -360,13 +359,18 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(MergeArgs a) {
 #pragma unroll
         for (int j = 0; j < 8; j++) {
             const uint32_t i = i0 + j * groups;
-            pre[j] = quad < quads ? *reinterpret_cast<const v4f*>(parts + (size_t)(i < active ? i : 0u) * stride + 4 + 4 * quad) : v4f{0.f, 0.f, 0.f, 0.f};
+            pre[j] = quad < quads ? *reinterpret_cast<const v4f*>(parts + (size_t)(i < a.splits ? i : 0u) * stride + 4 + 4 * quad) : v4f{0.f, 0.f, 0.f, 0.f};
         }
     };
     fetch(tid % cols, grp);
+    const float m_raw = parts[(size_t)(tid < a.splits ? tid : 0u) * stride], l_raw = parts[(size_t)(tid < a.splits ? tid : 0u) * stride + 1];
+    const uint32_t pos = (a.d_pos ? *a.d_pos : a.pos0) + t;
+    if (pos >= s.max_seq) return;
+    uint32_t active = pos / kChunk + 1u;  // what lies behind the active partials is from earlier steps: loaded, not used
+    active = active < a.splits ? active : a.splits;
     if (tid < 64) {
         const bool on = tid < active;
-        const float m_i = on ? parts[(size_t)tid * stride] : -__builtin_inff(), l_i = on ? parts[(size_t)tid * stride + 1] : 0.0f;
+        const float m_i = on ? m_raw : -__builtin_inff(), l_i = on ? l_raw : 0.0f;
         const float m = wave_max_f32(m_i), w = on ? expf(m_i - m) : 0.0f, l = wave_sum_f32(l_i * w);
         wts[tid] = w / l;
     }

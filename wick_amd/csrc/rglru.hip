@@ -143,14 +143,26 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(RecurrentStep a) {
     const uint16_t* row0 = row_of(part * kStepPart + grp);
     const uint32_t at0 = 8u * l < a.block ? 8u * l : 0u;
     const uint4 q0 = *reinterpret_cast<const uint4*>(row0 + at0), p0 = *reinterpret_cast<const uint4*>(row0 + (size_t)16 * a.gates.kp + at0);
+    // ... and so is what the first pass of channels needs behind it
+    const uint32_t ch0 = c0 + part * kStepPart + grp;
+    const float rb0 = a.r_bias[ch0], ib0 = a.i_bias[ch0], rate0 = a.rate[ch0], s0 = a.state[ch0], y0 = a.proj[ch0];
     for (uint32_t i = tid; i < a.block; i += 256) {
         const uint32_t ch = c0 + i;
         const float now = a.proj[a.channels + ch];
         float v = 0.0f;
-        for (uint32_t k = 0; k + 1 < a.taps; k++) {
-            const uint32_t back = a.taps - 1u - k;
-            const float tap = pos >= back ? a.ring[(size_t)((pos - back) % a.taps) * a.channels + ch] : 0.0f;
-            v += a.conv_w[(size_t)k * a.channels + ch] * tap;
+        if (a.taps <= 4u) {  // every tap's loads in flight together
+            float w[4], in[4];
+#pragma unroll
+            for (uint32_t m = 1; m < 4; m++) {
+                const bool on = m < a.taps;
+                w[m] = on ? a.conv_w[(size_t)(a.taps - 1u - m) * a.channels + ch] : 0.0f;
+                in[m] = on && pos >= m ? a.ring[(size_t)((pos - m) % a.taps) * a.channels + ch] : 0.0f;
+            }
+#pragma unroll
+            for (uint32_t m = 3; m > 0; m--) v += w[m] * in[m];
+        } else {
+            for (uint32_t m = a.taps - 1u; m > 0; m--)
+                v += a.conv_w[(size_t)(a.taps - 1u - m) * a.channels + ch] * (pos >= m ? a.ring[(size_t)((pos - m) % a.taps) * a.channels + ch] : 0.0f);
         }
         v += a.conv_w[(size_t)(a.taps - 1u) * a.channels + ch] * now;
         u[i] = v + a.conv_bias[ch];
@@ -175,11 +187,12 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(RecurrentStep a) {
         r = group_sum<LPR>(r), g = group_sum<LPR>(g);
         if (l == 0) {
             const uint32_t ch = c0 + f;
-            r = 1.0f / (1.0f + expf(-(r + a.r_bias[ch]))), g = 1.0f / (1.0f + expf(-(g + a.i_bias[ch])));
-            const float log_a = r * a.rate[ch], decay = expf(log_a);
-            const float s = decay * (pos > 0 ? a.state[ch] : 0.0f) + sqrtf(-expm1f(2.0f * log_a)) * (g * u[f]);
+            const bool first = f0 == 0;
+            r = 1.0f / (1.0f + expf(-(r + (first ? rb0 : a.r_bias[ch])))), g = 1.0f / (1.0f + expf(-(g + (first ? ib0 : a.i_bias[ch]))));
+            const float log_a = r * (first ? rate0 : a.rate[ch]), decay = expf(log_a);
+            const float s = decay * (pos == 0 ? 0.0f : first ? s0 : a.state[ch]) + sqrtf(-expm1f(2.0f * log_a)) * (g * u[f]);
             a.state[ch] = s;
-            a.out[ch] = s * a.proj[ch];
+            a.out[ch] = s * (first ? y0 : a.proj[ch]);
         }
     }
 }
