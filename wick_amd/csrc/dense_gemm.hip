@@ -93,6 +93,26 @@ struct EpiSilu {
         store4(out + (size_t)t * ldo + f, g);
     }
 };
+// Rows below `split` as they are, the pairs behind them through gelu(gate) * up.
+template <typename AT>
+struct EpiProject {
+    static constexpr bool kPaired = true, kTrans = false;
+    float* out;
+    uint32_t ldo, split;
+    AT* act;
+    uint32_t lda;
+    __device__ void operator()(uint32_t, uint32_t f, uint32_t t, v4f a, v4f b) const {
+        const uint32_t row = 2u * (f & ~15u) + (f & 15u);  // of the first of the two
+        if (row < split) {
+            float* o = out + (size_t)t * ldo + row;
+            store4(o, a), store4(o + 16, b);
+            return;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) a[i] = gelu_tanhf(a[i]) * b[i];
+        store4(act + (size_t)t * lda + (f - split / 2u), a);
+    }
+};
 template <typename AT>
 struct EpiConvert {
     static constexpr bool kPaired = false, kTrans = false;
@@ -373,6 +393,12 @@ hipError_t launch_gemm_silu(const DenseWeight& w, const GemmIn& in, void* out, u
     if (ldo < w.mp / 2u || ldo % 8u) return hipErrorInvalidValue;
     return in.f32 ? run_gemm(w, in, EpiSilu<float>{static_cast<float*>(out), ldo, row_scale}, L, g)
                   : run_gemm(w, in, EpiSilu<uint16_t>{static_cast<uint16_t*>(out), ldo, row_scale}, L, g);
+}
+
+hipError_t launch_gemm_project(const DenseWeight& w, const GemmIn& in, uint32_t split, float* out, uint32_t ldo, void* act, uint32_t lda, const Launch& L) {
+    if (split % kDensePad || split > w.mp || ldo < split || ldo % 4u || (split < w.mp && (!act || lda < (w.mp - split) / 2u || lda % 8u))) return hipErrorInvalidValue;
+    return in.f32 ? run_gemm(w, in, EpiProject<float>{out, ldo, split, static_cast<float*>(act), lda}, L)
+                  : run_gemm(w, in, EpiProject<uint16_t>{out, ldo, split, static_cast<uint16_t*>(act), lda}, L);
 }
 
 hipError_t launch_gemm_convert(const DenseWeight& w, const GemmIn& in, void* out, uint32_t ldo, bool transposed, const Launch& L) {

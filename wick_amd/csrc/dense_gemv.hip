@@ -43,7 +43,25 @@ __device__ __forceinline__ float block_sum_f32(float v, float* slots) {
     return (slots[0] + slots[1]) + (slots[2] + slots[3]);
 }
 
-enum { kProVec = 0, kProRow = 1, kProRowConv = 2, kProLoop = 3 };
+// Two sums in one exchange; slots: eight floats.
+__device__ __forceinline__ void block_sum2_f32(float& a, float& b, float* slots) {
+    a = wave_sum_f32(a), b = wave_sum_f32(b);
+    __syncthreads();
+    if ((threadIdx.x & 63u) == 0) slots[threadIdx.x >> 6] = a, slots[4 + (threadIdx.x >> 6)] = b;
+    __syncthreads();
+    a = (slots[0] + slots[1]) + (slots[2] + slots[3]), b = (slots[4] + slots[5]) + (slots[6] + slots[7]);
+}
+
+// Four floats at e of a row that ends at dim (zeros behind it); rows that end at a multiple of four are read as vectors.
+__device__ __forceinline__ v4f load_to(const float* p, uint32_t e, uint32_t dim) {
+    if (dim % 4u == 0) return *reinterpret_cast<const v4f*>(p + e);
+    v4f v;
+#pragma unroll
+    for (int i = 0; i < 4; i++) v[i] = e + i < dim ? p[e + i] : 0.0f;
+    return v;
+}
+
+enum { kProVec = 0, kProRow = 1, kProRowConv = 2, kProLoop = 3, kProGains = 4 };  // kProGains: a row stage with gains per coordinate
 
 // Fills vec[0 .. k): the vector itself, the row stage's h, or [x | 0 | x0 | 0].  All threads call it; it ends with a barrier.
 // A thread owns coordinates 4 t .. 4 t + 3 of every 1024: NQ vectors of four (dim <= 1024 NQ; rows are padded to 64).
@@ -58,6 +76,51 @@ __device__ __forceinline__ void fill_vector(const GemvIn& in, uint32_t k, float*
         }
         __syncthreads();
         return;
+    } else if constexpr (PRO == kProGains) {
+        const RowStage& s = in.row;
+        const v4f zero = {0.f, 0.f, 0.f, 0.f};
+        v4f x[NQ], y[NQ], y2[NQ], wn[NQ];
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const uint32_t e = 4u * (tid + kThreads * i);
+            const bool on = e < s.dim;
+            x[i] = on ? load_to(s.x, e, s.dim) : zero;
+            y[i] = on && s.y ? load_to(s.y, e, s.dim) : zero, y2[i] = on && s.y2 ? load_to(s.y2, e, s.dim) : zero;
+            wn[i] = on && s.w_pre ? load_to(s.w_pre, e, s.dim) : v4f{1.f, 1.f, 1.f, 1.f};
+            if (on && s.add) x[i] += load_to(s.add, e, s.dim);
+        }
+        if (s.y) {
+            v4f wp[NQ], wp2[NQ];
+            float ss = 0.0f, ss2 = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NQ; i++) {
+                const uint32_t e = 4u * (tid + kThreads * i);
+                wp[i] = e < s.dim && s.w_post ? load_to(s.w_post, e, s.dim) : v4f{1.f, 1.f, 1.f, 1.f};
+                wp2[i] = e < s.dim && s.w_post2 ? load_to(s.w_post2, e, s.dim) : v4f{1.f, 1.f, 1.f, 1.f};
+                ss += dot4(y[i], y[i]), ss2 += dot4(y2[i], y2[i]);
+            }
+            block_sum2_f32(ss, ss2, slots);
+            const float sy = s.g_post / sqrtf(ss / (float)s.dim + s.eps), sy2 = s.g_post / sqrtf(ss2 / (float)s.dim + s.eps);
+#pragma unroll
+            for (int i = 0; i < NQ; i++) {
+                x[i] += y[i] * wp[i] * sy;
+                if (s.y2) x[i] += y2[i] * wp2[i] * sy2;
+            }
+        }
+        float ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const uint32_t e = 4u * (tid + kThreads * i);
+            if (s.x_out && blockIdx.x == 0 && e < s.dim) *reinterpret_cast<v4f*>(s.x_out + e) = x[i];
+            ss += dot4(x[i], x[i]);
+        }
+        const float sx = s.g_pre / sqrtf(block_sum_f32(ss, slots) / (float)s.dim + s.eps);
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const uint32_t e = 4u * (tid + kThreads * i);
+            if (e < k) *reinterpret_cast<v4f*>(vec + e) = x[i] * wn[i] * sx;
+        }
+        __syncthreads();
     } else {
         const RowStage& s = in.row;
         const bool first = blockIdx.x == 0;
@@ -202,7 +265,7 @@ struct DenseArgs {
 template <int PRO, int NQ, int R>
 __global__ __launch_bounds__(256) void gemv_dense_kernel(DenseArgs a) {
     extern __shared__ __align__(16) float vec[];
-    __shared__ float slots[4];
+    __shared__ float slots[8];
     const uint32_t lane = threadIdx.x & 63u, row0 = (blockIdx.x * 4u + (threadIdx.x >> 6)) * R;
     const uint16_t* rows[R];
 #pragma unroll
@@ -223,6 +286,84 @@ __global__ __launch_bounds__(256) void gemv_dense_kernel(DenseArgs a) {
         if (a.act == kActGeluSplit && row < a.split) v = gelu_tanhf(v);
         if (a.act == kActRelu2) v = fmaxf(v, 0.0f), v = v * v;
         a.out[row] = v;
+    }
+}
+
+struct ProjectArgs {
+    const uint16_t* w;
+    uint32_t ldw, split, total, k;   // rows below split as they are, interleaved pairs up to total
+    GemvIn in;
+    float *out, *act;
+};
+
+// R rows a wave: R consecutive plain ones, or R / 2 pairs.
+template <int PRO, int NQ, int R>
+__global__ __launch_bounds__(256) void gemv_project_kernel(ProjectArgs a) {
+    extern __shared__ __align__(16) float vec[];
+    __shared__ float slots[8];
+    const uint32_t lane = threadIdx.x & 63u, row0 = (blockIdx.x * 4u + (threadIdx.x >> 6)) * R;
+    const bool pairs = row0 >= a.split;
+    const uint32_t f0 = (row0 - a.split) / 2u;  // the wave's first pair: R / 2 divides 16
+    const uint16_t* rows[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const uint32_t f = f0 + r / 2, row = pairs ? a.split + (f >> 4) * 32u + (f & 15u) + 16u * (r & 1) : row0 + r;
+        rows[r] = a.w + (size_t)(row < a.total ? row : a.total - 1u) * a.ldw;
+    }
+    Ahead<R> ahead;
+    ahead.load(rows, a.k);
+    fill_vector<PRO, NQ>(a.in, a.k, vec, slots);
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = 0.0f;
+    dot_rows<R, true>(rows, &ahead, vec, a.k, acc);
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = wave_sum_f32(acc[r]);
+    if (lane != 0 || row0 >= a.total) return;
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        if (!pairs) a.out[row0 + r] = acc[r];
+        else if (r % 2 == 0) a.act[f0 + r / 2] = gelu_tanhf(acc[r]) * acc[r + 1];
+    }
+}
+
+struct SegmentArgs {
+    GemvSegment s[kMaxSegments];
+    uint32_t first[kMaxSegments + 1];  // workgroups of segment i: first[i] .. first[i + 1] - 1
+    uint32_t count;
+};
+
+template <int R>
+__global__ __launch_bounds__(256) void gemv_segments_kernel(SegmentArgs a) {
+    extern __shared__ __align__(16) float vec[];  // [k] | [parts]
+    uint32_t i = 0;
+    while (i + 1 < a.count && blockIdx.x >= a.first[i + 1]) i++;
+    const GemvSegment& s = a.s[i];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, k = s.w.kp, row0 = ((blockIdx.x - a.first[i]) * 4u + (tid >> 6)) * R;
+    const uint16_t* rows[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) rows[r] = s.w.d + (size_t)(row0 + r < s.m ? row0 + r : s.m - 1u) * k;
+    Ahead<R> ahead;
+    ahead.load(rows, k);
+    for (uint32_t e = 4u * tid; e < k; e += 4u * kThreads) {
+        v4f v = {0.f, 0.f, 0.f, 0.f};
+        if (e < s.vec_len) v = load_to(s.vec, e, s.vec_len);
+        *reinterpret_cast<v4f*>(vec + e) = v;
+    }
+    if (s.norm_w) {
+        part_rms(vec, s.vec_len, s.parts, s.eps, vec + k);
+        const uint32_t len = s.vec_len / s.parts;
+        for (uint32_t e = tid; e < s.vec_len; e += kThreads) vec[e] *= vec[k + e / len] * s.norm_w[e];
+    }
+    __syncthreads();
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = 0.0f;
+    dot_rows<R, true>(rows, &ahead, vec, k, acc);
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        const float v = wave_sum_f32(acc[r]);
+        if (lane == 0 && row0 + r < s.m) s.out[row0 + r] = v;
     }
 }
 
@@ -370,7 +511,42 @@ hipError_t launch_gemv_dense(const DenseWeight& w, uint32_t m, const GemvIn& in,
         if (in.x0_at != pad_to(in.row.dim, kDensePad) || 2u * in.x0_at != a.k) return hipErrorInvalidValue;
         return run_dense_nq<kProLoop>(a, L);
     }
+    if (in.row.vector_gains()) return in.row.conv ? hipErrorInvalidValue : run_dense_nq<kProGains>(a, L);
     return in.row.conv ? run_dense_nq<kProRowConv>(a, L) : run_dense_nq<kProRow>(a, L);
+}
+
+hipError_t launch_gemv_project(const DenseWeight& w, uint32_t split, const GemvIn& in, float* out, float* act, const Launch& L) {
+    const ProjectArgs a{w.d, w.kp, split, w.mp, w.kp, in, out, act};
+    if (!w.d || !out || split % kDensePad || split > w.mp || (split < w.mp && !act) || a.k > kGemvMaxK || in.vec || in.x0 || in.row.conv || !row_ok(in.row, a.k))
+        return hipErrorInvalidValue;
+    constexpr uint32_t R = 4;
+    const dim3 grid(w.mp / (4u * R));
+    const uint32_t lds = a.k * 4u, dim = in.row.dim;
+    if (dim <= 1024u) return launch_kernel_lds(L, kFamGemv, gemv_project_kernel<kProGains, 1, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 2048u) return launch_kernel_lds(L, kFamGemv, gemv_project_kernel<kProGains, 2, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 4096u) return launch_kernel_lds(L, kFamGemv, gemv_project_kernel<kProGains, 4, R>, grid, dim3(kThreads), lds, a);
+    if (dim <= 8192u) return launch_kernel_lds(L, kFamGemv, gemv_project_kernel<kProGains, 8, R>, grid, dim3(kThreads), lds, a);
+    return hipErrorInvalidValue;
+}
+
+hipError_t launch_gemv_segments(const GemvSegment* segs, uint32_t count, const Launch& L) {
+    if (count == 0 || count > kMaxSegments) return hipErrorInvalidValue;
+    SegmentArgs a{};
+    a.count = count;
+    uint32_t lds = 0, rows = 0;
+    for (uint32_t i = 0; i < count; i++) rows += segs[i].m;
+    const uint32_t R = rows <= 1024u ? 1 : 2;
+    for (uint32_t i = 0; i < count; i++) {
+        const GemvSegment& s = a.s[i] = segs[i];
+        if (!s.w.d || !s.vec || !s.out || s.m == 0 || s.m > s.w.mp || s.vec_len > s.w.kp || s.w.kp % 8u || s.w.kp > kGemvMaxK || s.parts == 0 || s.vec_len % s.parts ||
+            s.parts > 512u)
+            return hipErrorInvalidValue;
+        a.first[i + 1] = a.first[i] + (s.m + 4u * R - 1u) / (4u * R);
+        const uint32_t need = (s.w.kp + s.parts) * 4u;
+        lds = need > lds ? need : lds;
+    }
+    return R == 1 ? launch_kernel_lds(L, kFamGemv, gemv_segments_kernel<1>, dim3(a.first[count]), dim3(kThreads), lds, a)
+                  : launch_kernel_lds(L, kFamGemv, gemv_segments_kernel<2>, dim3(a.first[count]), dim3(kThreads), lds, a);
 }
 
 uint32_t routed_act_floats(const RoutedMlp& m) { return m.top * (m.gate_up.mp / 2u) + (m.shared_gate_up.d ? m.shared_gate_up.mp / 2u : 0u) + 4u; }

@@ -31,6 +31,7 @@ struct FolderModelClass {
 };
 
 int load_lokinex(wick_rocm_ctx* ctx, const wick_safetensors* folder, int dtype, uint32_t context_size, wick_rocm_model** out);
+int load_zirurax(wick_rocm_ctx* ctx, const wick_safetensors* folder, int dtype, uint32_t context_size, wick_rocm_model** out);
 
 // One step of a model on the context's stream: a replay of the graph in `slot` (captured when there is none yet, or when the
 // context's scratch moved since), or, without `use_graph` or while per-dispatch timing is on, the launches of `enqueue` one by one.

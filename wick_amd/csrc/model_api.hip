@@ -9,6 +9,7 @@ namespace {
 // The architectures config.json may name.
 constexpr FolderModelClass kFolderModels[] = {
     {"Lokinex", load_lokinex},
+    {"Zirurax", load_zirurax},
 };
 constexpr uint32_t kFolderModelCount = sizeof(kFolderModels) / sizeof(kFolderModels[0]);
 

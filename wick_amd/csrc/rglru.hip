@@ -5,59 +5,40 @@
 // (chunk, channel) first reduces its tokens to one affine map, then starts from the maps of the chunks before it.  A decode step
 // does everything between the block's projections in one launch.
 #include "wick_rocm_dense.h"
+#include "short_conv.h"
 #include "wick_rocm_device.h"
 
 namespace wick_rocm {
 
 namespace {
 
-constexpr uint32_t kConvTokens = 8;    // tokens per thread of the prompt convolution; at least taps - 1
 constexpr uint32_t kScanChunk = 32;
 
 __device__ __forceinline__ void put(float* p, float v) { *p = v; }
 __device__ __forceinline__ void put(uint16_t* p, float v) { *p = __builtin_bit_cast(uint16_t, (__bf16)v); }
 
-// One thread: one channel, kConvTokens tokens, their inputs and the ones in front of them in registers (FAST: up to four taps).
-// Only the threads of the first tokens read the ring, and they alone write it, after their reads.
-template <bool FAST, typename AT>
-__global__ __launch_bounds__(256) void recurrent_conv_kernel(RecurrentConv a, uint32_t n) {
-    constexpr int BACK = FAST ? 3 : (int)kConvTokens;
-    const uint32_t ch = blockIdx.x * 256u + threadIdx.x, t0 = blockIdx.y * kConvTokens;
-    if (ch >= a.channels) return;
-    const float* x = a.proj + a.x_at + ch;
-    const uint32_t block = ch / a.block, terms = sizeof(AT) == 2 ? 2u : 1u;
-    AT* ua = static_cast<AT*>(a.ua) + (size_t)block * terms * a.block + ch % a.block;
-    const float bias = a.bias[ch];
-    float in[BACK + (int)kConvTokens], w[BACK + 1];  // w by distance: the newest input is the last tap
+// u as f32 rows and in the activation type of the gates' product (bfloat16: two terms).
+template <typename AT>
+struct ConvToGates {
+    float* u;
+    AT* ua;
+    uint32_t channels, block, lda;
+    __device__ void operator()(uint32_t ch, uint32_t t0, const float (&v)[kConvTokens], uint32_t count) const {
+        const uint32_t terms = sizeof(AT) == 2 ? 2u : 1u;
+        AT* o = ua + (size_t)(ch / block) * terms * block + ch % block + (size_t)t0 * lda;
 #pragma unroll
-    for (int i = 0; i < BACK + (int)kConvTokens; i++) {
-        const int t = (int)t0 + i - BACK, p = (int)a.pos0 + t;
-        in[i] = 0.0f;
-        if (t >= 0) in[i] = x[(size_t)(t < (int)n ? t : (int)n - 1) * a.ldp];
-        else if (p >= 0 && BACK - i < (int)a.taps) in[i] = a.ring[(size_t)((uint32_t)p % a.taps) * a.channels + ch];
-    }
-#pragma unroll
-    for (int m = 0; m <= BACK; m++) w[m] = m < (int)a.taps ? a.w[(size_t)(a.taps - 1u - m) * a.channels + ch] : 0.0f;
-#pragma unroll
-    for (int i = 0; i < (int)kConvTokens; i++) {
-        const uint32_t t = t0 + i;
-        if (t >= n) break;
-        float v = 0.0f;
-#pragma unroll
-        for (int m = BACK; m >= 0; m--) v += w[m] * in[i + BACK - m];
-        v += bias;
-        a.u[(size_t)t * a.channels + ch] = v;
-        AT* o = ua + (size_t)t * a.lda;
-        if constexpr (sizeof(AT) == 2) {
-            const float hi = (float)(__bf16)v;
-            put(o, hi), put(o + a.block, v - hi);
-        } else {
-            put(o, v);
+        for (uint32_t i = 0; i < kConvTokens; i++, o += lda) {
+            if (i >= count) break;
+            u[(size_t)(t0 + i) * channels + ch] = v[i];
+            if constexpr (sizeof(AT) == 2) {
+                const float hi = (float)(__bf16)v[i];
+                put(o, hi), put(o + block, v[i] - hi);
+            } else {
+                put(o, v[i]);
+            }
         }
     }
-    if (blockIdx.y == 0)
-        for (uint32_t t = n > a.taps ? n - a.taps : 0u; t < n; t++) a.ring[(size_t)((a.pos0 + t) % a.taps) * a.channels + ch] = x[(size_t)t * a.ldp];
-}
+};
 
 // Scratch: [chunks][channels] products of a, the same of the chunk's own result, [channels] the state the portion starts from.
 // The first chunk's result already contains that state.
@@ -202,13 +183,9 @@ __global__ __launch_bounds__(256) void recurrent_step_kernel(RecurrentStep a) {
 hipError_t launch_recurrent_conv(const RecurrentConv& a, uint32_t n, const Launch& L) {
     if (n == 0) return hipSuccess;
     if (a.taps == 0 || a.taps > kConvTokens || a.block == 0 || a.channels % a.block || a.lda < a.channels * (a.f32 ? 1u : 2u)) return hipErrorInvalidValue;
-    const dim3 grid((a.channels + 255u) / 256u, (n + kConvTokens - 1u) / kConvTokens);
-    auto go = [&](auto fast) {
-        constexpr bool F = decltype(fast)::value;
-        return a.f32 ? launch_kernel(L, kFamOther, recurrent_conv_kernel<F, float>, grid, dim3(256), a, n)
-                     : launch_kernel(L, kFamOther, recurrent_conv_kernel<F, uint16_t>, grid, dim3(256), a, n);
-    };
-    return a.taps <= 4u ? go(std::integral_constant<bool, true>{}) : go(std::integral_constant<bool, false>{});
+    const ShortConv c{a.proj + a.x_at, a.ldp, a.channels, a.taps, a.pos0, a.w, a.bias, a.ring};
+    return a.f32 ? launch_short_conv(c, n, n, ConvToGates<float>{a.u, static_cast<float*>(a.ua), a.channels, a.block, a.lda}, L)
+                 : launch_short_conv(c, n, n, ConvToGates<uint16_t>{a.u, static_cast<uint16_t*>(a.ua), a.channels, a.block, a.lda}, L);
 }
 
 size_t recurrent_scan_scratch_floats(uint32_t n, uint32_t channels) { return ((size_t)2 * ((n + kScanChunk - 1u) / kScanChunk) + 1u) * channels; }

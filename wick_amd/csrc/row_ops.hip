@@ -34,32 +34,38 @@ __device__ __forceinline__ float row_y(const RowStage& s, uint32_t t, uint32_t e
     return v;
 }
 
-// One row by the calling wave: dst[0 .. dim) = x + g_post y / rms(y), normed when NORM.  dst may be LDS or global memory; a lane
+// One row by the calling wave: dst[0 .. dim) = the updated residual, normed when NORM.  dst may be LDS or global memory; a lane
 // only re-reads what it wrote itself.
 template <bool NORM>
 __device__ __forceinline__ void stage_row(const RowStage& s, uint32_t t, float* dst, float* x_out) {
     const uint32_t lane = threadIdx.x & 63u;
     const float* x = s.x + (size_t)t * s.x_stride;
+    const float *y2 = s.y2 ? s.y2 + (size_t)t * s.y_stride : nullptr, *add = s.add ? s.add + (size_t)t * s.y_stride : nullptr;
     const bool has_y = s.y || s.experts;
-    float sy = 0.0f;
+    float sy = 0.0f, sy2 = 0.0f;
     if (has_y) {
-        float ss = 0.0f;
+        float ss = 0.0f, ss2 = 0.0f;
         for (uint32_t e = lane; e < s.dim; e += 64) {
             const float v = row_y(s, t, e);
             ss += v * v;
+            if (y2) ss2 += y2[e] * y2[e];
         }
         sy = s.g_post / sqrtf(wave_sum_f32(ss) / (float)s.dim + s.eps);
+        if (y2) sy2 = s.g_post / sqrtf(wave_sum_f32(ss2) / (float)s.dim + s.eps);
     }
     float ss = 0.0f;
     for (uint32_t e = lane; e < s.dim; e += 64) {
-        const float v = has_y ? x[e] + row_y(s, t, e) * sy : x[e];
+        float v = x[e];
+        if (has_y) v += row_y(s, t, e) * sy * (s.w_post ? s.w_post[e] : 1.0f);
+        if (y2) v += y2[e] * sy2 * (s.w_post2 ? s.w_post2[e] : 1.0f);
+        if (add) v += add[e];
         dst[e] = v;
         if (x_out) x_out[e] = v;
         ss += v * v;
     }
     if constexpr (NORM) {
         const float sx = s.g_pre / sqrtf(wave_sum_f32(ss) / (float)s.dim + s.eps);
-        for (uint32_t e = lane; e < s.dim; e += 64) dst[e] *= sx;
+        for (uint32_t e = lane; e < s.dim; e += 64) dst[e] *= s.w_pre ? sx * s.w_pre[e] : sx;
     }
 }
 
@@ -134,6 +140,12 @@ __device__ __forceinline__ v4f mask4(v4f v, uint32_t e, uint32_t dim) {
         if (e + i >= dim) v[i] = 0.0f;
     return v;
 }
+__device__ __forceinline__ v4f load_gain(const float* w, uint32_t e, uint32_t dim) {  // (a gain's row ends at dim)
+    v4f v;
+#pragma unroll
+    for (int i = 0; i < 4; i++) v[i] = e + i < dim ? w[e + i] : 0.0f;
+    return v;
+}
 __device__ __forceinline__ float dot4(v4f a, v4f b) { return (a[0] * b[0] + a[1] * b[1]) + (a[2] * b[2] + a[3] * b[3]); }
 
 // sum[r] over the workgroup for R values per thread.  red: [R][NT / 64].
@@ -156,23 +168,34 @@ __device__ __forceinline__ void block_sums(float (&v)[R], float* red) {
     }
 }
 
-// Rows first .. first + R - 1 (clamped to n - 1; negative ones are left at zero): h[r] = x + g_post y / rms(y), normed when NORM;
-// rows from `own` on are stored to x_out.
-template <bool NORM, int R, int NT>
+// Rows first .. first + R - 1 (clamped to n - 1; negative ones are left at zero): h[r] = the updated residual, normed when NORM;
+// rows from `own` on are stored to x_out.  GAINS: gains per coordinate, the second normed and the plain addend.
+template <bool NORM, bool GAINS, int R, int NT>
 __device__ __forceinline__ void stage_tile(const RowsArgs& a, int first, int own, v4f (&h)[R], float* red) {
     const RowStage& s = a.s;
     const uint32_t e = 4u * threadIdx.x;
     const bool on = e < s.dim, has_y = s.y || s.experts;
-    v4f y[R];
+    v4f y[R], y2[GAINS ? R : 1], add[GAINS ? R : 1];
+    v4f wp, wp2, wn;
     uint32_t row[R];
+    if constexpr (GAINS) {
+        const v4f one = {1.f, 1.f, 1.f, 1.f};
+        wp = on && s.w_post ? load_gain(s.w_post, e, s.dim) : one, wp2 = on && s.w_post2 ? load_gain(s.w_post2, e, s.dim) : one;
+        wn = on && s.w_pre ? load_gain(s.w_pre, e, s.dim) : one;
+    }
 #pragma unroll
     for (int r = 0; r < R; r++) {
         const int j = first + r < (int)a.n ? first + r : (int)a.n - 1;
         row[r] = j < 0 ? 0u : a.rows ? a.rows[j] : (uint32_t)j;
         h[r] = y[r] = v4f{0.f, 0.f, 0.f, 0.f};
+        if constexpr (GAINS) y2[r] = add[r] = v4f{0.f, 0.f, 0.f, 0.f};
         if (!on || first + r < 0) continue;
         h[r] = load4(s.x + (size_t)row[r] * s.x_stride + e);
         if (s.y) y[r] = load4(s.y + (size_t)row[r] * s.y_stride + e);
+        if constexpr (GAINS) {
+            if (s.y2) y2[r] = load4(s.y2 + (size_t)row[r] * s.y_stride + e);
+            if (s.add) add[r] = load4(s.add + (size_t)row[r] * s.y_stride + e);
+        }
     }
     if (s.experts) {
         const float share = 1.0f / (float)s.top;
@@ -186,7 +209,24 @@ __device__ __forceinline__ void stage_tile(const RowsArgs& a, int first, int own
         }
     }
     float ss[R];
-    if (has_y) {
+    if constexpr (GAINS) {
+        if (has_y) {
+            float both[2 * R];
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                y[r] = mask4(y[r], e, s.dim), y2[r] = mask4(y2[r], e, s.dim);
+                both[r] = dot4(y[r], y[r]), both[R + r] = dot4(y2[r], y2[r]);
+            }
+            block_sums<2 * R, NT>(both, red);
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                h[r] += y[r] * wp * (s.g_post / sqrtf(both[r] / (float)s.dim + s.eps));
+                if (s.y2) h[r] += y2[r] * wp2 * (s.g_post / sqrtf(both[R + r] / (float)s.dim + s.eps));
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < R; r++) h[r] += add[r];
+    } else if (has_y) {
 #pragma unroll
         for (int r = 0; r < R; r++) y[r] = mask4(y[r], e, s.dim), ss[r] = dot4(y[r], y[r]);
         block_sums<R, NT>(ss, red);
@@ -204,13 +244,17 @@ __device__ __forceinline__ void stage_tile(const RowsArgs& a, int first, int own
         block_sums<R, NT>(ss, red);
 #pragma unroll
         for (int r = 0; r < R; r++) h[r] *= s.g_pre / sqrtf(ss[r] / (float)s.dim + s.eps);
+        if constexpr (GAINS) {
+#pragma unroll
+            for (int r = 0; r < R; r++) h[r] *= wn;
+        }
     }
 }
 
-template <int MODE, bool CONV, int R, int NT, typename AT>
+template <int MODE, bool CONV, bool GAINS, int R, int NT, typename AT>
 __global__ __launch_bounds__(NT) void rows_fast_kernel(RowsArgs a) {
     constexpr int HALO = CONV ? kHalo : 0, TILE = R - HALO;
-    __shared__ float red[R * (NT / 64)];
+    __shared__ float red[(GAINS ? 2 : 1) * R * (NT / 64)];
     const RowStage& s = a.s;
     const uint32_t e = 4u * threadIdx.x;
     const int j0 = (int)blockIdx.x * TILE;
@@ -220,7 +264,7 @@ __global__ __launch_bounds__(NT) void rows_fast_kernel(RowsArgs a) {
         for (int m = 0; m <= kHalo; m++)  // by distance: the newest input is the last tap
             w[m] = m < (int)s.taps && e < s.dim ? mask4(load4(s.conv + (size_t)(s.taps - 1u - m) * s.x_stride + e), e, s.dim) : v4f{0.f, 0.f, 0.f, 0.f};
     }
-    stage_tile<MODE == kRowNorm, R, NT>(a, j0 - HALO, HALO, h, red);
+    stage_tile<MODE == kRowNorm, GAINS, R, NT>(a, j0 - HALO, HALO, h, red);
     if constexpr (MODE == kRowOnly) return;
     if constexpr (CONV) {
         if (j0 == 0) {  // the inputs in front of this portion
@@ -271,7 +315,7 @@ __global__ __launch_bounds__(NT) void rows_fast_kernel(RowsArgs a) {
             v4f tail[kHalo + 1];
             RowsArgs b = a;
             b.s.x_out = nullptr;
-            stage_tile<true, kHalo + 1, NT>(b, (int)a.n - kHalo - 1, kHalo + 1, tail, red);
+            stage_tile<true, GAINS, kHalo + 1, NT>(b, (int)a.n - kHalo - 1, kHalo + 1, tail, red);
 #pragma unroll
             for (int r = 0; r <= kHalo; r++) {
                 const int j = (int)a.n - kHalo - 1 + r;
@@ -283,17 +327,32 @@ __global__ __launch_bounds__(NT) void rows_fast_kernel(RowsArgs a) {
 }
 
 template <typename AT>
-__global__ __launch_bounds__(256) void embed_activation_kernel(const uint16_t* __restrict__ embed, uint32_t vocab, uint32_t dim,
+__global__ __launch_bounds__(256) void embed_activation_kernel(const uint16_t* __restrict__ embed, uint32_t vocab, uint32_t dim, float scale,
                                                                const uint32_t* __restrict__ tokens, float* __restrict__ x, uint32_t x_stride,
                                                                AT* __restrict__ xa, uint32_t ldo, uint32_t kp) {
     const uint32_t t = blockIdx.x, token = tokens[t];
     const uint16_t* row = embed + (size_t)(token < vocab ? token : 0u) * dim;  // the host refuses tokens past the vocabulary
     const uint32_t width = xa ? kp : dim;
     for (uint32_t e = threadIdx.x; e < width; e += 256) {
-        const float v = e < dim ? __uint_as_float((uint32_t)row[e] << 16) : 0.0f;
+        const float v = e < dim ? __uint_as_float((uint32_t)row[e] << 16) * scale : 0.0f;
         if (e < dim) x[(size_t)t * x_stride + e] = v;
         if (xa) put(xa + (size_t)t * ldo + e, v);
     }
+}
+
+// One row per workgroup, in LDS meanwhile: every part's sum of squares by one wave (few parts: by the whole workgroup).
+template <typename AT>
+__global__ __launch_bounds__(256) void part_norm_kernel(const float* __restrict__ y, uint32_t ldy, uint32_t dim, uint32_t parts, const float* __restrict__ w,
+                                                        float eps, AT* __restrict__ out, uint32_t ldo, uint32_t kp) {
+    extern __shared__ __align__(16) float row[];  // [dim] | [parts]
+    float* inv = row + dim;
+    const uint32_t tid = threadIdx.x;
+    const float* src = y + (size_t)blockIdx.x * ldy;
+    for (uint32_t e = tid; e < dim; e += 256) row[e] = src[e];
+    __syncthreads();
+    part_rms(row, dim, parts, eps, inv);
+    const uint32_t len = dim / parts;
+    for (uint32_t e = tid; e < kp; e += 256) put(out + (size_t)blockIdx.x * ldo + e, e < dim ? row[e] * inv[e / len] * w[e] : 0.0f);
 }
 
 // One workgroup per table: counts per expert, their running sums and tiles, then every pair to its entry.  The order of an
@@ -342,14 +401,18 @@ template <int MODE, bool CONV, typename AT>
 hipError_t run_rows(const RowsArgs& a, const Launch& L) {
     const uint32_t kp = MODE == kRowOnly ? a.s.dim : a.kp;
     const bool aligned = a.s.x_stride % 4u == 0 && (a.s.y_stride % 4u == 0) && a.ldo % 4u == 0 && a.lo_at % 4u == 0 && kp <= pad_to(a.s.dim, kDensePad) &&
-                         pad_to(a.s.dim, kDensePad) <= a.s.x_stride && (!(a.s.y || a.s.experts) || pad_to(a.s.dim, kDensePad) <= a.s.y_stride);
+                         pad_to(a.s.dim, kDensePad) <= a.s.x_stride && (!a.s.pending() || pad_to(a.s.dim, kDensePad) <= a.s.y_stride);
     if (aligned && kp <= 4096u && (!CONV || a.s.taps <= (uint32_t)kHalo + 1u)) {
-        constexpr int R = CONV ? 11 : 4;
-        const dim3 grid((a.n + R - (CONV ? kHalo : 0) - 1) / (R - (CONV ? kHalo : 0)));
-        if (kp <= 1024u) return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, R, 256, AT>, grid, dim3(256), a);
-        if (kp <= 2048u) return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, R, 512, AT>, grid, dim3(512), a);
-        return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, CONV ? 7 : 4, 1024, AT>,
-                             CONV ? dim3((a.n + 3u) / 4u) : grid, dim3(1024), a);
+        auto go = [&](auto gains) {
+            constexpr bool G = decltype(gains)::value;
+            constexpr int R = CONV ? 11 : 4;
+            const dim3 grid((a.n + R - (CONV ? kHalo : 0) - 1) / (R - (CONV ? kHalo : 0)));
+            if (kp <= 1024u) return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, G, R, 256, AT>, grid, dim3(256), a);
+            if (kp <= 2048u) return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, G, R, 512, AT>, grid, dim3(512), a);
+            return launch_kernel(L, kFamOther, rows_fast_kernel<MODE, CONV, G, CONV ? 7 : 4, 1024, AT>, CONV ? dim3((a.n + 3u) / 4u) : grid, dim3(1024), a);
+        };
+        if (!a.s.vector_gains()) return go(std::false_type{});
+        if constexpr (!CONV) return go(std::true_type{});  // (with a convolution: the general form)
     }
     const uint32_t halo = CONV ? a.s.taps - 1u : 0u;
     uint32_t tile = 8;
@@ -376,7 +439,7 @@ hipError_t launch_rows(const RowsArgs& a, int mode, const Launch& L) {
     if (a.n == 0) return hipSuccess;
     const bool conv = a.s.conv != nullptr;
     if (!a.s.x || a.s.dim == 0 || a.s.x_stride < a.s.dim || (mode != kRowOnly && (!a.out || a.kp < a.s.dim || a.ldo < a.kp)) || (conv && (a.rows || !a.s.ring || a.s.taps == 0)) ||
-        (mode != kRowNorm && conv) || (mode == kRowOnly && !a.s.x_out) || a.s.x_out == a.s.x)
+        (mode != kRowNorm && conv) || (mode == kRowOnly && !a.s.x_out) || a.s.x_out == a.s.x || (a.s.y2 && !a.s.y))
         return hipErrorInvalidValue;
     if (mode == kRowNorm) {
         if (conv) return a.f32 ? run_rows<kRowNorm, true, float>(a, L) : run_rows<kRowNorm, true, uint16_t>(a, L);
@@ -386,12 +449,21 @@ hipError_t launch_rows(const RowsArgs& a, int mode, const Launch& L) {
     return run_rows<kRowOnly, false, float>(a, L);
 }
 
-hipError_t launch_embed_activation(const uint16_t* embed, uint32_t vocab, uint32_t dim, const uint32_t* tokens, uint32_t n, float* x, uint32_t x_stride, void* xa,
+hipError_t launch_part_norm(const float* y, uint32_t ldy, uint32_t n, uint32_t dim, uint32_t parts, const float* w, float eps, void* out, uint32_t ldo, uint32_t kp,
+                            bool f32, const Launch& L) {
+    if (n == 0) return hipSuccess;
+    if (parts == 0 || dim % parts || kp < dim || ldo < kp || ldy < dim || (size_t)(dim + parts) * 4u > 64u * 1024u) return hipErrorInvalidValue;
+    const uint32_t lds = (dim + parts) * 4u;
+    return f32 ? launch_kernel_lds(L, kFamOther, part_norm_kernel<float>, dim3(n), dim3(256), lds, y, ldy, dim, parts, w, eps, static_cast<float*>(out), ldo, kp)
+               : launch_kernel_lds(L, kFamOther, part_norm_kernel<uint16_t>, dim3(n), dim3(256), lds, y, ldy, dim, parts, w, eps, static_cast<uint16_t*>(out), ldo, kp);
+}
+
+hipError_t launch_embed_activation(const uint16_t* embed, uint32_t vocab, uint32_t dim, float scale, const uint32_t* tokens, uint32_t n, float* x, uint32_t x_stride, void* xa,
                                    uint32_t ldo, uint32_t kp, bool f32, const Launch& L) {
     if (n == 0) return hipSuccess;
     if (x_stride < dim || (xa && (kp < dim || ldo < kp))) return hipErrorInvalidValue;
-    return f32 ? launch_kernel(L, kFamOther, embed_activation_kernel<float>, dim3(n), dim3(256), embed, vocab, dim, tokens, x, x_stride, static_cast<float*>(xa), ldo, kp)
-               : launch_kernel(L, kFamOther, embed_activation_kernel<uint16_t>, dim3(n), dim3(256), embed, vocab, dim, tokens, x, x_stride,
+    return f32 ? launch_kernel(L, kFamOther, embed_activation_kernel<float>, dim3(n), dim3(256), embed, vocab, dim, scale, tokens, x, x_stride, static_cast<float*>(xa), ldo, kp)
+               : launch_kernel(L, kFamOther, embed_activation_kernel<uint16_t>, dim3(n), dim3(256), embed, vocab, dim, scale, tokens, x, x_stride,
                                static_cast<uint16_t*>(xa), ldo, kp);
 }
 

@@ -106,6 +106,7 @@ struct EmbedArgs {
     float* out;
     int type;
     uint32_t m, k;
+    float scale;  // of a looked-up row
 };
 
 // Row `row` of the embedding into emb.out by the calling workgroup, four elements per thread at a time: their loads are all issued
@@ -121,7 +122,7 @@ __device__ __forceinline__ void embed_row_batched(const EmbedArgs& emb, uint32_t
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             const uint32_t e = e0 + j * blockDim.x;
-            if (e < emb.k) emb.out[e] = v[j];
+            if (e < emb.k) emb.out[e] = __fmul_rn(v[j], emb.scale);
         }
     }
 }
@@ -204,24 +205,25 @@ hipError_t launch_embed_rows(const uint8_t* d_w, int type, uint32_t m, uint32_t 
 
 hipError_t launch_argmax(const float* d_x, uint32_t n, unsigned long long* d_partial, uint32_t* d_out, uint32_t* d_token, uint32_t* d_pos,
                          uint32_t* d_history, uint32_t history_len, const Launch& L, const uint8_t* d_embd, int embd_type, uint32_t embd_m,
-                         uint32_t embd_k, float* d_embd_out) {
+                         uint32_t embd_k, float* d_embd_out, float embd_scale) {
     const uint32_t blocks = n >= 4096u ? kArgmaxBlocks : 1u;
     hipError_t e = launch_kernel(L, kFamOther, argmax_partial_kernel, dim3(blocks), dim3(256), d_x, n, d_partial);
     if (e != hipSuccess) return e;
-    return launch_argmax_final(d_partial, blocks, n, d_out, d_token, d_pos, d_history, history_len, L, d_embd, embd_type, embd_m, embd_k, d_embd_out);
+    return launch_argmax_final(d_partial, blocks, n, d_out, d_token, d_pos, d_history, history_len, L, d_embd, embd_type, embd_m, embd_k, d_embd_out,
+                               embd_scale);
 }
 
 hipError_t launch_argmax_final(const unsigned long long* d_partial, uint32_t n_partials, uint32_t n, uint32_t* d_out, uint32_t* d_token, uint32_t* d_pos,
                                uint32_t* d_history, uint32_t history_len, const Launch& L, const uint8_t* d_embd, int embd_type, uint32_t embd_m,
-                               uint32_t embd_k, float* d_embd_out) {
-    const EmbedArgs emb{d_embd_out ? d_embd : nullptr, d_embd_out, embd_type, embd_m, embd_k};
+                               uint32_t embd_k, float* d_embd_out, float embd_scale) {
+    const EmbedArgs emb{d_embd_out ? d_embd : nullptr, d_embd_out, embd_type, embd_m, embd_k, embd_scale};
     return launch_kernel(L, kFamOther, argmax_final_kernel, dim3(1), dim3(emb.w || n_partials > 64u ? 256 : 64), d_partial, n_partials, n, d_out, d_token,
                          d_pos, d_history, history_len, emb);
 }
 
 hipError_t launch_set_step(uint32_t* d_token, uint32_t token, uint32_t* d_pos, uint32_t pos, const Launch& L, const uint8_t* d_embd, int embd_type,
-                           uint32_t embd_m, uint32_t embd_k, float* d_embd_out) {
-    const EmbedArgs emb{d_embd_out ? d_embd : nullptr, d_embd_out, embd_type, embd_m, embd_k};
+                           uint32_t embd_m, uint32_t embd_k, float* d_embd_out, float embd_scale) {
+    const EmbedArgs emb{d_embd_out ? d_embd : nullptr, d_embd_out, embd_type, embd_m, embd_k, embd_scale};
     return launch_kernel(L, kFamOther, set_step_kernel, dim3(1), dim3(256), d_token, token, d_pos, pos, emb);
 }
 

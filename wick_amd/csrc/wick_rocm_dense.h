@@ -41,6 +41,13 @@ struct RowStage {
     const float* experts = nullptr;     // [n * top][y_stride]
     const uint32_t* slots = nullptr;    // [n][top]: the entry that holds expert s of token t
     uint32_t top = 0;
+    // gains per coordinate, and the outputs of sublayers that read the same norm: x_out = x + g_post * (w_post * y / rms(y)
+    // + w_post2 * y2 / rms(y2)) + add, h = g_pre * w_pre * x_out / rms(x_out)
+    const float *w_pre = nullptr, *w_post = nullptr;    // [dim]; null: ones
+    const float *y2 = nullptr, *w_post2 = nullptr;      // [n][y_stride], [dim]; y2 needs y
+    const float* add = nullptr;                         // [n][y_stride]
+    __host__ __device__ bool pending() const { return y || experts || add; }
+    __host__ __device__ bool vector_gains() const { return w_pre || w_post || y2 || add; }
 };
 
 // ---- matrix products of a prompt (dense_gemm.hip) ---------------------------------------------------------------------------
@@ -71,6 +78,9 @@ hipError_t launch_gemm_relu2(const DenseWeight& w, const GemmIn& in, void* out, 
 // out[t][f] = silu(gate) * up (* row_scale[t]) of an interleaved weight, in the activation type.
 hipError_t launch_gemm_silu(const DenseWeight& w, const GemmIn& in, void* out, uint32_t ldo, const float* row_scale, const Launch& L,
                             const Grouping& g = Grouping());
+// Several projections of one input in one product: rows below `split` (a multiple of 64) are stored as f32, out[t][f]; the interleaved
+// pairs behind them become act[t][j] = gelu_tanh(gate) * up in the activation type.
+hipError_t launch_gemm_project(const DenseWeight& w, const GemmIn& in, uint32_t split, float* out, uint32_t ldo, void* act, uint32_t lda, const Launch& L);
 // out[t][f] = W x in the activation type, or transposed: out[f][t] (ldo >= n rounded up to 4).
 hipError_t launch_gemm_convert(const DenseWeight& w, const GemmIn& in, void* out, uint32_t ldo, bool transposed, const Launch& L);
 // The gates of a real-gated linear recurrence, block-diagonal: per block b an interleaved weight over the block's columns of x;
@@ -95,6 +105,21 @@ struct GemvIn {
     const uint32_t* d_pos = nullptr;
 };
 hipError_t launch_gemv_dense(const DenseWeight& w, uint32_t m, const GemvIn& in, float* out, const float* bias, int act, uint32_t split, const Launch& L);
+// The step's counterpart of launch_gemm_project: out[f] below `split`, act[j] behind it.
+hipError_t launch_gemv_project(const DenseWeight& w, uint32_t split, const GemvIn& in, float* out, float* act, const Launch& L);
+// Up to kMaxSegments products of their own vectors in one launch; with norm_w the vector is first normed in `parts` equal parts.
+struct GemvSegment {
+    DenseWeight w;
+    uint32_t m;
+    const float* vec;
+    uint32_t vec_len;              // floats of vec (zeros are taken behind them)
+    float* out;
+    const float* norm_w = nullptr; // [vec_len]
+    uint32_t parts = 1;
+    float eps = 0.0f;
+};
+constexpr uint32_t kMaxSegments = 4;
+hipError_t launch_gemv_segments(const GemvSegment* segs, uint32_t count, const Launch& L);
 // Routed gated feed-forward of one token: act_e[s][ffp] = silu(gate) * up of expert table[token][s], act_s[..] of the shared one,
 // shared_gate[0] = sigmoid(w_sg . h).
 struct RoutedMlp {
@@ -129,8 +154,11 @@ struct RowsArgs {
 };
 hipError_t launch_rows(const RowsArgs& a, int mode, const Launch& L);
 uint32_t rows_max_dim(uint32_t taps);
-// Embedding rows -> x f32 [n][x_stride] and, when given, the activation form at xa [n][ldo] (kp columns).
-hipError_t launch_embed_activation(const uint16_t* embed, uint32_t vocab, uint32_t dim, const uint32_t* tokens, uint32_t n, float* x, uint32_t x_stride, void* xa,
+// out[t] = w * y[t] / rms in `parts` equal parts of the row, in the activation type (kp columns, zeros behind dim).
+hipError_t launch_part_norm(const float* y, uint32_t ldy, uint32_t n, uint32_t dim, uint32_t parts, const float* w, float eps, void* out, uint32_t ldo, uint32_t kp,
+                            bool f32, const Launch& L);
+// Embedding rows * scale -> x f32 [n][x_stride] and, when given, the activation form at xa [n][ldo] (kp columns).
+hipError_t launch_embed_activation(const uint16_t* embed, uint32_t vocab, uint32_t dim, float scale, const uint32_t* tokens, uint32_t n, float* x, uint32_t x_stride, void* xa,
                                    uint32_t ldo, uint32_t kp, bool f32, const Launch& L);
 // Groups the n * top (token, expert) pairs of one table by expert: entry_token[e], slot_of[t][s], tiles of kGroupTileRows entries.
 struct RouteJob {
@@ -211,5 +239,73 @@ hipError_t launch_latent_attention(const LatentShape& s, const LatentWeights& w,
 bool latent_prefill_shape(uint32_t dim, uint32_t rot, uint32_t vdim, uint32_t* dqp, uint32_t* dvp);
 hipError_t launch_latent_prefill(const LatentShape& s, const uint16_t* q, const uint16_t* kx, uint32_t ldk, const uint16_t* vt, uint32_t ldv, uint32_t dqp,
                                  uint32_t dvp, uint32_t n, uint32_t pos0, uint16_t* out, uint32_t ldo, uint32_t kp, const Launch& L);
+
+// ---- grouped-query attention over a window (windowed_attention.hip) ---------------------------------------------------------------
+// Position i sees j with i - window < j <= i (window 0: every j <= i); query head h uses key / value head h / (heads / kv_heads);
+// scores are capped, the weighted values gated: out = sigmoid(gate) * sum.  The cache is a ring of `slots` positions, a multiple of 64
+// that holds a window and a portion: keys [slots][kv_heads][dqp], values in tiles of 64 positions [slots / 64][kv_heads][dvp][64],
+// zeros behind dim / vdim; bfloat16, or f32.
+struct WindowShape {
+    uint32_t heads, kv_heads, dim, vdim;
+    uint32_t dqp, dvp;           // multiples of 32
+    uint32_t rot;                // coordinates of a head that turn, in pairs (2i, 2i + 1); even
+    uint32_t window, slots, max_seq;
+    float scale, softcap;        // softcap 0: none
+    bool f32;                    // element type of the cache
+};
+// Columns of a projection [n][ldp]: q [heads][dqp], k [kv_heads][dqp], v [kv_heads][dvp], g [heads][dvp]; multiples of 4.
+struct WindowProj {
+    const float* p;
+    uint32_t ldp, q_at, k_at, v_at, g_at;
+    const float* rope;           // [max_seq][rot / 2][2]: cosine, sine
+};
+uint32_t window_slots(uint32_t window, uint32_t portion, uint32_t max_seq);
+bool window_prefill_shape(uint32_t dim, uint32_t vdim);   // dqp / dvp of the next function have matrix-core kernels
+void window_pads(uint32_t dim, uint32_t vdim, uint32_t* dqp, uint32_t* dvp);
+size_t window_attention_scratch_floats(const WindowShape& s, uint32_t n);
+// Keys (rotated) and values of n tokens into the cache.
+hipError_t launch_window_store(const WindowShape& s, const WindowProj& w, void* kc, void* vc, uint32_t n, uint32_t pos0, const Launch& L);
+// n tokens over the cache, all arithmetic f32: out[t][h * vdim ..] f32 or the activation form (kp columns).  With d_pos: one token at
+// *d_pos whose key and value are not in the cache yet; they are appended.
+hipError_t launch_window_attention(const WindowShape& s, const WindowProj& w, void* kc, void* vc, float* scratch, uint32_t n, uint32_t pos0,
+                                   const uint32_t* d_pos, void* out, uint32_t ldo, uint32_t kp, bool out_f32, const Launch& L);
+// A prompt's queries on the matrix cores (bfloat16 cache, window_prefill_shape).
+hipError_t launch_window_prefill(const WindowShape& s, const WindowProj& w, const void* kc, const void* vc, uint32_t n, uint32_t pos0, uint16_t* out,
+                                 uint32_t ldo, uint32_t kp, const Launch& L);
+
+// ---- state-space duality (ssd.hip) --------------------------------------------------------------------------------------------------
+// Per head a state S [vdim][state]: S_t = exp(rate dt_t) S_(t-1) + dt_t x_t B_t^T, y_t = S_t C_t + D x_t, out = y * silu(z); x, B, C
+// behind a short convolution with silu, dt = softplus(. + dt_bias).  Channels of the convolution: [x: heads * pp | B: groups * np |
+// C: groups * np], vdim and state padded with zero channels.
+struct SsdShape {
+    uint32_t heads, groups, state, vdim, taps;
+    uint32_t np, pp;             // state to a power of two >= 32, vdim to a multiple of 16
+    __host__ __device__ uint32_t channels() const { return heads * pp + 2u * groups * np; }
+};
+struct SsdWeights {
+    const float *conv, *conv_bias;          // [taps][channels], [channels]
+    const float *rate, *dt_bias, *d;        // [heads]; rate = -exp(A_log)
+};
+// Columns of a projection [n][ldp]: z [heads][pp], the convolution's channels at x_at, dt [heads].
+struct SsdProj {
+    const float* p;
+    uint32_t ldp, z_at, x_at, dt_at;
+};
+constexpr uint32_t kSsdMaxState = 512;
+// One token: convolution, state and gate; out [heads * vdim] f32.
+hipError_t launch_ssd_step(const SsdShape& s, const SsdWeights& w, const SsdProj& p, float* ring, float* state, float* out, const uint32_t* d_pos, const Launch& L);
+// A portion, token by token in f32 (rows: [n][channels] scratch).  out [n][ldo] f32.
+hipError_t launch_ssd_scan(const SsdShape& s, const SsdWeights& w, const SsdProj& p, float* ring, float* state, float* rows, uint32_t n, uint32_t pos0,
+                           float* out, uint32_t ldo, const Launch& L);
+// A portion in chunks of 64 tokens on the matrix cores.
+struct SsdScratch {
+    uint16_t *tiles, *rows;      // [chunks][heads * pp + groups * np][64], [chunks * 64][2 * groups * np]
+    float* meta;                 // [chunks][heads][2][64] | [chunks][heads]
+    float* sums;                 // [chunks][heads * pp * np]: a chunk's own contribution to the state
+    uint16_t* starts;            // [chunks][heads][2][pp * np]: the state in front of a chunk, hi | lo
+};
+inline uint32_t ssd_chunks(uint32_t n) { return (n + 63u) / 64u; }
+hipError_t launch_ssd_chunks(const SsdShape& s, const SsdWeights& w, const SsdProj& p, float* ring, float* state, const SsdScratch& scratch, uint32_t n,
+                             uint32_t pos0, float* out, uint32_t ldo, const Launch& L);
 
 }  // namespace wick_rocm

@@ -231,6 +231,32 @@ __device__ __forceinline__ float wave_max_f32(float v) {
     return fmaxf(fmaxf(r0, r1), fmaxf(r2, r3));
 }
 
+// inv[i] = 1 / rms of part i of a row in LDS (`parts` equal parts), by a workgroup of 256 threads; begins and ends with a barrier.
+__device__ __forceinline__ void part_rms(const float* row, uint32_t dim, uint32_t parts, float eps, float* inv) {
+    __shared__ float slots[4];
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, len = dim / parts;
+    __syncthreads();
+    if (parts < 4u) {
+        for (uint32_t i = 0; i < parts; i++) {
+            float ss = 0.0f;
+            for (uint32_t e = tid; e < len; e += 256) ss += row[i * len + e] * row[i * len + e];
+            ss = wave_sum_f32(ss);
+            if (lane == 0) slots[wave] = ss;
+            __syncthreads();
+            if (tid == 0) inv[i] = 1.0f / sqrtf(((slots[0] + slots[1]) + (slots[2] + slots[3])) / (float)len + eps);
+            __syncthreads();
+        }
+        return;
+    }
+    for (uint32_t i = wave; i < parts; i += 4) {
+        float ss = 0.0f;
+        for (uint32_t e = lane; e < len; e += 64) ss += row[i * len + e] * row[i * len + e];
+        ss = wave_sum_f32(ss);
+        if (lane == 0) inv[i] = 1.0f / sqrtf(ss / (float)len + eps);
+    }
+    __syncthreads();
+}
+
 // Reductions over the four lane groups of a query (lanes l, l ^ 16, l ^ 32, l ^ 48) with gfx950's row / half swaps: swapping a
 // register with a copy of itself leaves the two partners' values in the pair, so their maximum (or sum) needs no select
 // and no trip through the LDS crossbar.  Every lane ends with the result.

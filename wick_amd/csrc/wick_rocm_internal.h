@@ -226,16 +226,16 @@ hipError_t launch_silu_mul(float* d_gate, const float* d_up, uint32_t n, const L
 // d_history[pos] = pick (pos = *d_pos before it is advanced), when given.  d_partial: scratch of kArgmaxPartials keys, 8-byte aligned;
 // d_x 16-byte aligned.
 constexpr uint32_t kArgmaxPartials = 4096;  // 64 for the two-stage pick; up to one key per wave of a Q6_K LM head that leaves its own
-// d_embd_out non-null: the pick's row of the embedding (d_embd, type, m x k) is written there as the next step's input.
+// d_embd_out non-null: the pick's row of the embedding (d_embd, type, m x k), times embd_scale, is written there as the next step's input.
 hipError_t launch_argmax(const float* d_x, uint32_t n, unsigned long long* d_partial, uint32_t* d_out, uint32_t* d_token, uint32_t* d_pos,
                          uint32_t* d_history, uint32_t history_len, const Launch& L, const uint8_t* d_embd = nullptr, int embd_type = 0,
-                         uint32_t embd_m = 0, uint32_t embd_k = 0, float* d_embd_out = nullptr);
+                         uint32_t embd_m = 0, uint32_t embd_k = 0, float* d_embd_out = nullptr, float embd_scale = 1.0f);
 // The second stage on its own, over n_partials keys that a producer has left in d_partial (n = the number of candidates; 0: pick 0).
 hipError_t launch_argmax_final(const unsigned long long* d_partial, uint32_t n_partials, uint32_t n, uint32_t* d_out, uint32_t* d_token, uint32_t* d_pos,
                                uint32_t* d_history, uint32_t history_len, const Launch& L, const uint8_t* d_embd = nullptr, int embd_type = 0,
-                               uint32_t embd_m = 0, uint32_t embd_k = 0, float* d_embd_out = nullptr);
+                               uint32_t embd_m = 0, uint32_t embd_k = 0, float* d_embd_out = nullptr, float embd_scale = 1.0f);
 hipError_t launch_set_step(uint32_t* d_token, uint32_t token, uint32_t* d_pos, uint32_t pos, const Launch& L, const uint8_t* d_embd = nullptr,
-                           int embd_type = 0, uint32_t embd_m = 0, uint32_t embd_k = 0, float* d_embd_out = nullptr);
+                           int embd_type = 0, uint32_t embd_m = 0, uint32_t embd_k = 0, float* d_embd_out = nullptr, float embd_scale = 1.0f);
 hipError_t launch_advance_pos(uint32_t* d_pos, const Launch& L);
 
 // n at and above which gemm_q8 uses the MFMA kernel (when k % 128 == 0): the counterpart of GEMM_MIN_N = 16
