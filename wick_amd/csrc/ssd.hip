@@ -186,7 +186,10 @@ struct ConvToTiles {
         if (ch < xs + gn) *reinterpret_cast<bf8*>(tiles + ((size_t)(t0 / kChunk) * (xs + gn) + ch) * kChunk + t0 % kChunk) = b;
         if (ch >= xs) {
 #pragma unroll
-            for (uint32_t i = 0; i < kConvTokens; i++) rows[(size_t)(t0 + i) * 2u * gn + ch - xs] = __builtin_bit_cast(uint16_t, b[i]);
+            for (uint32_t i = 0; i < kConvTokens; i++) {
+                const __bf16 one = b[i];
+                rows[(size_t)(t0 + i) * 2u * gn + ch - xs] = __builtin_bit_cast(uint16_t, one);
+            }
         }
     }
 };

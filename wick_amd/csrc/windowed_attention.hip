@@ -453,15 +453,16 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(PrefillArgs a) {
         for (int i = 0; i < NV; i++) {
             const uint32_t d = 16 * i + 4 * g;
             const v4f z = *reinterpret_cast<const v4f*>(gate + d);
-            bf4 b;
+            v4f y;
 #pragma unroll
-            for (int r = 0; r < 4; r++) b[r] = (__bf16)(o[i][r] * inv / (1.0f + expf(-z[r])));
+            for (int r = 0; r < 4; r++) y[r] = o[i][r] * inv / (1.0f + expf(-z[r]));
             if (s.vdim % 4u == 0) {
+                const bf4 b = {(__bf16)y[0], (__bf16)y[1], (__bf16)y[2], (__bf16)y[3]};
                 if (d < s.vdim) *reinterpret_cast<bf4*>(out + d) = b;
             } else {
 #pragma unroll
                 for (int r = 0; r < 4; r++)
-                    if (d + r < s.vdim) out[d + r] = __builtin_bit_cast(uint16_t, b[r]);
+                    if (d + r < s.vdim) put(out + d + r, y[r]);
             }
         }
         if (h + 1 == s.heads)
