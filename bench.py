@@ -781,19 +781,29 @@ LOKINEX_SIZES = {"350m": dict(D=1024, heads=16, rank=256, dense_ff=6912, expert_
                  "1p2b": dict(D=2048, heads=32, rank=512, dense_ff=10368, expert_ff=2048, experts=8, top=2, shared_ff=2816)}
 
 
-def lokinex_folder(path, D, heads, rank, dense_ff, expert_ff, experts, top, shared_ff, moe, vocab=VOCAB):
-    """A randomly initialised model folder (values drawn once per 4 M and repeated: the kernels' time does not depend on them)."""
-    from wick_amd.checkpoint import to_bf16, write_folder
+class FolderWriter:
+    """Tensors of a randomly initialised model folder (values drawn once per 4 M and repeated: the kernels' time does not depend on them)."""
 
-    rng = np.random.default_rng(7)
-    base = rng.standard_normal(1 << 22).astype(np.float32)
-    t = {}
+    def __init__(self):
+        self.rng = np.random.default_rng(7)
+        self.base = self.rng.standard_normal(1 << 22).astype(np.float32)
+        self.t = {}
 
-    def put(name, shape, sigma, center=0.0):
+    def put(self, name, shape, sigma, center=0.0):
+        from wick_amd.checkpoint import to_bf16
+
         n = int(np.prod(shape))
-        t[name] = np.resize(to_bf16(center + sigma * base[:min(n, base.size)]), n).reshape(shape)
+        self.t[name] = np.resize(to_bf16(center + sigma * self.base[:min(n, self.base.size)]), n).reshape(shape)
 
-    mat = lambda name, m, k: put(name, (m, k), k ** -0.5)
+    def mat(self, name, m, k):
+        self.put(name, (m, k), k ** -0.5)
+
+
+def lokinex_folder(path, D, heads, rank, dense_ff, expert_ff, experts, top, shared_ff, moe, vocab=VOCAB):
+    from wick_amd.checkpoint import write_folder
+
+    w = FolderWriter()
+    rng, t, put, mat = w.rng, w.t, w.put, w.mat
     layers = []
     for i in range(14):
         p, x, f = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
@@ -831,16 +841,53 @@ def lokinex_folder(path, D, heads, rank, dense_ff, expert_ff, experts, top, shar
                         "loop": {"start": 6, "stop": 8, "times": 2}}, t)
 
 
-def bench_lokinex(ctx, W, O, size="350m", moe=True, context=4096, tokens=64, trace=False, prompts=(512, 2002)):
-    """Decode steps and prompt passes of the Lokinex model handle, measured like bench_lfm2_step's."""
+# Zirurax at the sizes of LFM2-350M / -1.2B (hidden, heads, key / value width, vocabulary, 16 layers) with feed-forwards that make a token's
+# weights about Lokinex's.
+ZIRURAX_SIZES = {"350m": dict(D=1024, heads=16, kv_heads=8, ff=3456), "1p2b": dict(D=2048, heads=32, kv_heads=8, ff=5120)}
+
+
+def zirurax_folder(path, D, heads, kv_heads, ff, window=1024, state=128, vocab=VOCAB):
+    from wick_amd.checkpoint import write_folder
+
+    w = FolderWriter()
+    put, mat = w.put, w.mat
+    layers = []
+    for i in range(16):
+        p, x, y, f = f"l{i}.", f"l{i}.mix.left.", f"l{i}.mix.right.", f"l{i}.mlp."
+        for n in (p + "norm1", x + "out", y + "out", y + "norm"):
+            put(n, (D,), 0.0, 1.0)
+        mat(x + "q", heads * 64, D), mat(x + "k", kv_heads * 64, D), mat(x + "v", kv_heads * 64, D), mat(x + "g", heads * 64, D), mat(x + "o", D, heads * 64)
+        ssd = D // 64
+        mat(y + "in", 2 * D + 2 * state + ssd, D), mat(y + "o", D, D)
+        put(y + "conv", (D + 2 * state, 4), 0.5), put(y + "conv.b", (D + 2 * state,), 0.1)
+        put(y + "dt_bias", (ssd,), 1.0, -3.0), put(y + "A_log", (ssd,), 0.5), put(y + "D", (ssd,), 0.1, 1.0)
+        mat(f + "gate", ff, D), mat(f + "up", ff, D), mat(f + "down", D, ff)
+        left = {"heads": heads, "kv_heads": kv_heads, "dim": 64, "vdim": 64, "scale": 0.125, "softcap": 30.0, "mask": {"size": window},
+                "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+        right = {"heads": ssd, "groups": 1, "state": state, "vdim": 64, "conv": 4, "norm_groups": 1}
+        layers.append({"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": {"kind": "dense", "ff": ff}})
+    mat("embed", vocab, D), put("final.norm", (D,), 0.0, 1.0)
+    write_folder(path, {"architecture": "Zirurax", "vocab": vocab, "width": D, "embedding": {"scale": float(D) ** 0.5}, "norm": {"eps": 1e-6}, "layers": layers}, w.t)
+
+
+def bench_lokinex(ctx, W, O, size="350m", moe=True, **kw):
+    return bench_folder(ctx, f"Lokinex {size}, {'routed' if moe else 'dense'} feed-forwards", lambda d: lokinex_folder(d, moe=moe, **LOKINEX_SIZES[size]), **kw)
+
+
+def bench_zirurax(ctx, W, O, size="350m", **kw):
+    return bench_folder(ctx, f"Zirurax {size}, window 1024", lambda d: zirurax_folder(d, **ZIRURAX_SIZES[size]), **kw)
+
+
+def bench_folder(ctx, label, write, context=4096, tokens=64, trace=False, prompts=(512, 2002)):
+    """Decode steps and prompt passes of a folder model's handle, measured like bench_lfm2_step's."""
     import tempfile
 
     from wick_amd.model import RocmModel
 
     with tempfile.TemporaryDirectory() as d:
-        lokinex_folder(d, moe=moe, **LOKINEX_SIZES[size])
+        write(d)
         model = RocmModel(ctx, d, context)
-    out = {"model": f"Lokinex {size}, {'routed' if moe else 'dense'} feed-forwards, {model.layer_runs} layer runs, bf16, random init", "context": context,
+    out = {"model": f"{label}, {model.layer_runs} layer runs, bf16, random init", "context": context,
            "gpu_memory_MB": model.gpu_memory_bytes() / 1e6, "runs": [], "prefill": []}
     if trace:  # eager launches for a kernel tracer: 16 steps from position 1024, two prompt passes
         model.set_graph_replay(False)
@@ -891,6 +938,12 @@ def bench_lokinex_all(ctx, W, O):
             "lfm2_1p2b_q8": bench_lfm2_step(ctx, W, O, body=8, embd=8, dims=big, label="LFM2-1.2B-shaped")}
 
 
+def bench_zirurax_all(ctx, W, O):
+    """The design beside the closest model the library had (Lokinex, bf16) at equal hidden size, heads, vocabulary and layer runs."""
+    return {"zirurax_350m": bench_zirurax(ctx, W, O, "350m"), "lokinex_350m_dense": bench_lokinex(ctx, W, O, "350m", moe=False),
+            "zirurax_1p2b": bench_zirurax(ctx, W, O, "1p2b"), "lokinex_1p2b_dense": bench_lokinex(ctx, W, O, "1p2b", moe=False)}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -901,7 +954,7 @@ def main():
     ap.add_argument("--prompt-tokens", type=int, default=2002, help="lfm2_prefill_trace: tokens of the traced prompt pass")
     ap.add_argument("--graph-only", action="store_true", help="decode legs: graph replays only, no eager launches (for kernel tracers)")
     ap.add_argument("--mfma-shape", type=int, default=0, help="block loop of the wide GEMM tile: 0 / 32 (default) or 16 (A/B runs)")
-    ap.add_argument("--leg", default="all", help="all | c1 | gemm | decode | decode_q8 | gemv | prefill_sites | lm_head | lm_head_q6k | upload | lfm2_step | lfm2_step_q8 | lfm2_step_kv16 | lfm2_step_1p2b | lfm2_step_trace | lfm2_prefill_trace | lokinex | lokinex_350m | lokinex_trace | lfm2_q8_trace | copy | probe | cpu")
+    ap.add_argument("--leg", default="all", help="all | c1 | gemm | decode | decode_q8 | gemv | prefill_sites | lm_head | lm_head_q6k | upload | lfm2_step | lfm2_step_q8 | lfm2_step_kv16 | lfm2_step_1p2b | lfm2_step_trace | lfm2_prefill_trace | lokinex | lokinex_350m | lokinex_trace | zirurax | zirurax_350m | zirurax_trace | lfm2_q8_trace | copy | probe | cpu")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on ONE GPU only (no collectives, no sharding); use --gpus 1", file=sys.stderr)
@@ -936,6 +989,9 @@ def main():
             "lfm2_step_trace": lambda: trace_lfm2_step(ctx, W, O),
             "lfm2_prefill_trace": lambda: trace_lfm2_prefill(ctx, W, O, n=args.prompt_tokens),
             # another architecture at equal sizes, and its eager launches for a kernel tracer
+            "zirurax": lambda: bench_zirurax_all(ctx, W, O),
+            "zirurax_350m": lambda: bench_zirurax(ctx, W, O, "350m"),
+            "zirurax_trace": lambda: bench_zirurax(ctx, W, O, "350m", trace=True),
             "lokinex": lambda: bench_lokinex_all(ctx, W, O),
             "lokinex_350m": lambda: bench_lokinex(ctx, W, O, "350m"),
             "lokinex_trace": lambda: bench_lokinex(ctx, W, O, "350m", trace=True),

@@ -35,6 +35,8 @@ def frequencies(rot):
 
 def rope_partial(v, pos, rot):
     """Turns the pairs (2i, 2i + 1) of the first rot.dims coordinates of v [T, heads, dim]; the others pass."""
+    if not rot:
+        return v
     out = v.copy()
     a = pos[:, None, None] * frequencies(rot)
     u, w = v[..., 0:rot["dims"]:2], v[..., 1:rot["dims"]:2]
@@ -47,8 +49,8 @@ def windowed_attention(h, t, p, m, pos, cache, r=exact):
     """Grouped-query attention over the last mask.size positions, capped scores, gated output.  cache: (keys, values) of every position
     before h[0]."""
     n, H, G, dim, vdim = len(h), m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q = rope_partial((r(h) @ t[p + "q"].T).reshape(n, H, dim), pos, m["rot"])
-    k = rope_partial((r(h) @ t[p + "k"].T).reshape(n, G, dim), pos, m["rot"])
+    q = rope_partial((r(h) @ t[p + "q"].T).reshape(n, H, dim), pos, m.get("rot"))
+    k = rope_partial((r(h) @ t[p + "k"].T).reshape(n, G, dim), pos, m.get("rot"))
     v = (r(h) @ t[p + "v"].T).reshape(n, G, vdim)
     gate = sigmoid(r(h) @ t[p + "g"].T)
     k, v = np.concatenate([cache[0], r(k)]), np.concatenate([cache[1], r(v)])

@@ -3,16 +3,16 @@
 The f32 model is held to f32 rounding, which shows a wrong key, a lost state or a tap that is off by one anywhere; the served
 (bfloat16) model to three times what rounding the products' activations does to the plain implementation on the same tokens.  Where random weights would hide a fault -- one far key among hundreds -- the
 weights are made so that the fault would move the logits by far more than the tolerance, and the test says so first."""
-import json
-import os
 import subprocess
 import sys
 
 import numpy as np
 import pytest
 
+import folder_pair
 import lokinex_synth as S
 from conftest import ROOT
+from folder_pair import TOL_F32, error, greedy, run_trace
 from oracle import lokinex_oracle as O
 from wick_amd import model as M
 from wick_amd.checkpoint import from_bf16, to_bf16
@@ -21,58 +21,11 @@ from wick_amd.rocm import RocmError
 
 pytestmark = pytest.mark.gpu
 
-TOL_F32 = 2e-5
 BOTH = pytest.mark.parametrize("dtype", [F32, NATIVE], ids=["f32", "bf16"])
 
 
-def error(got, want):
-    """Per row: rms of the difference over the rms of what is expected, the worst row."""
-    got, want = np.atleast_2d(got).astype(np.float64), np.atleast_2d(want).astype(np.float64)
-    assert got.shape == want.shape and np.isfinite(got).all()
-    return float(np.max(np.sqrt(np.mean((got - want) ** 2, -1) / np.mean(want ** 2, -1))))
-
-
-class Pair:
-    """A model on the GPU and its oracle."""
-
-    def __init__(self, ctx, tmp_path, cfg, dtype, seed=1, context=320, t=None):
-        self.cfg, self.dtype = cfg, dtype
-        self.t = S.tensors(cfg, seed) if t is None else t
-        self.path = S.write(tmp_path / f"m{seed}", cfg, self.t)
-        self.gpu = RocmModel(ctx, self.path, context, dtype)
-        self.oracle = O.LokinexOracle(cfg, self.t)
-        self.rounded = O.LokinexOracle(cfg, self.t, r=O.bfloat16)
-        self.tol = TOL_F32
-
-    def tokens(self, n, seed=0):
-        return np.random.default_rng(seed).integers(0, self.cfg["vocab"], n)
-
-    def want(self, toks, trace=None):
-        """What is expected for toks; sets the tolerance that `check` uses from here on."""
-        self.oracle.reset()
-        want = self.oracle.forward(toks, trace)
-        if self.dtype == NATIVE:
-            self.rounded.reset()
-            self.tol = 3.0 * error(self.rounded.forward(toks), want)
-        return want
-
-    def check(self, got, want):
-        e = error(got, want)
-        assert e <= self.tol, f"error {e:.2e}, tolerance {self.tol:.2e}"
-
-    def portions(self, toks, cuts):
-        got, at = [], 0
-        for c in cuts:
-            got.append(self.gpu.forward(toks[at:at + c], at, np.arange(c)))
-            at += c
-        assert at == len(toks)
-        return np.concatenate(got)
-
-    def __enter__(self):
-        return self
-
-    def __exit__(self, *exc):
-        self.gpu.free()
+def Pair(ctx, tmp_path, cfg, dtype, **kw):
+    return folder_pair.Pair(ctx, tmp_path, S, O.LokinexOracle, cfg, dtype, **kw)
 
 
 # One mechanism at a time, then together; sizes that the kernels have to pad, values of 1, the shapes that take other routes.
@@ -308,15 +261,6 @@ def test_graph_replay_is_the_same_launches(ctx, tmp_path, dtype):
             ctx.sync()
 
 
-def greedy(p, prompt, n):
-    p.oracle.reset()
-    logits, out = p.oracle.forward(prompt)[-1], []
-    for _ in range(n):
-        out.append(M.greedy_pick(logits))
-        logits = p.oracle.forward([out[-1]])[-1]
-    return out
-
-
 def test_greedy_generation(ctx, tmp_path):
     """The generation loop over the handle: chunked prompt, picks on the device, stop tokens, a sampler in their place."""
     with Pair(ctx, tmp_path, S.mixed(), F32, seed=13) as p:
@@ -343,13 +287,6 @@ def test_cancel_between_chunks(ctx, tmp_path):
         done, logits = p.gpu.prefill_chunked(toks[6:], 6, 6)
         assert done == 14
         p.check(logits, p.want(toks)[-1])
-
-
-def run_trace(path, dtype, steps, out, max_tokens):
-    proc = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", path, "--dtype", dtype, "--out", str(out), "--max-tokens", str(max_tokens)],
-                          input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=100)
-    assert proc.returncode == 0, proc.stderr[-2000:]
-    return [l for l in proc.stdout.splitlines() if l.startswith("done ")]
 
 
 @pytest.mark.parametrize("dtype, kind", [("float32", F32), ("bfloat16", NATIVE)])

@@ -36,7 +36,7 @@ def test_round_trip(tmp_path):
 
 
 def test_registry_names_the_architecture():
-    assert "Lokinex" in M.folder_architectures()
+    assert {"Lokinex", "Zirurax"} <= set(M.folder_architectures())
 
 
 def test_escapes_and_metadata(tmp_path):
