@@ -161,10 +161,9 @@ struct TileAt {
     uint32_t m0, t0, rows, z;   // first feature, first output row, rows present, block
     const uint16_t* w;
 };
-__device__ __forceinline__ bool tile_at(const GemmArgs& a, uint32_t bm, uint32_t bn, TileAt& o) {
-    uint32_t bid = blockIdx.x;
+__device__ __forceinline__ bool tile_at(const GemmArgs& a, uint32_t bm, uint32_t bn, uint32_t bid, uint32_t count, TileAt& o) {
     // consecutive workgroups go to the eight XCDs in turn: give every XCD a contiguous run of tiles
-    if (gridDim.x % 8u == 0) bid = (bid & 7u) * (gridDim.x >> 3) + (bid >> 3);
+    if (count % 8u == 0) bid = (bid & 7u) * (count >> 3) + (bid >> 3);
     const uint32_t mtiles = (a.mp + bm - 1) / bm;
     const uint32_t nt = bid / mtiles;
     o.m0 = (bid % mtiles) * bm, o.z = blockIdx.z;
@@ -218,13 +217,14 @@ __device__ __forceinline__ void run_epilogue(const GemmArgs& a, const TileAt& o,
     }
 }
 
+// Tile `bid` of `count`.
 template <int MT, int NT, int PD, class Epi>
-__global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
+__device__ __forceinline__ void gemm_bf16_tile(const GemmArgs& a, const Epi& epi, uint32_t bid, uint32_t count) {
     constexpr uint32_t BM = 32 * MT, BN = 32 * NT, BK = 64;
     constexpr int LA = BM * 8 / 256, LB = BN * 8 / 256;  // 16-byte chunks per thread and step
     __shared__ __align__(16) uint16_t sa[2][BM * BK], sb[2][BN * BK];
     TileAt o;
-    if (!tile_at(a, BM, BN, o)) return;
+    if (!tile_at(a, BM, BN, bid, count, o)) return;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, g = lane >> 4;
     const uint32_t wm = (wave & 1u) * (16 * MT), wn = (wave >> 1) * (16 * NT);
     const uint16_t* x = static_cast<const uint16_t*>(a.x) + (size_t)o.z * a.x_stride_z;
@@ -300,13 +300,30 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
     run_epilogue<MT, NT>(a, o, epi, acc, wm, wn, l16, g);
 }
 
+template <int MT, int NT, int PD, class Epi>
+__global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
+    gemm_bf16_tile<MT, NT, PD>(a, epi, blockIdx.x, gridDim.x);
+}
+
+struct StoresArgs {
+    GemmArgs a[kMaxStores];
+    EpiStore e[kMaxStores];
+    uint32_t first[kMaxStores + 1], count;  // tiles of product i: first[i] .. first[i + 1] - 1
+};
+template <int MT, int NT, int PD>
+__global__ __launch_bounds__(256) void gemm_bf16_stores_kernel(StoresArgs s) {
+    uint32_t i = 0;
+    while (i + 1 < s.count && blockIdx.x >= s.first[i + 1]) i++;
+    gemm_bf16_tile<MT, NT, PD>(s.a[i], s.e[i], blockIdx.x - s.first[i], s.first[i + 1] - s.first[i]);
+}
+
 template <class Epi>
 __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs a, Epi epi) {
     constexpr int MT = 2, NT = 2;
     constexpr uint32_t BM = 64, BN = 64, BK = 32, LD = BK + 4;
     __shared__ __align__(16) float sa[BM * LD], sb[BN * LD];
     TileAt o;
-    if (!tile_at(a, BM, BN, o)) return;
+    if (!tile_at(a, BM, BN, blockIdx.x, gridDim.x, o)) return;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, g = lane >> 4;
     const uint32_t wm = (wave & 1u) * 32u, wn = (wave >> 1) * 32u;
     const float* x = static_cast<const float*>(a.x) + (size_t)o.z * a.x_stride_z;
@@ -376,6 +393,42 @@ hipError_t run_gemm(const DenseWeight& w, const GemmIn& in, const Epi& epi, cons
 hipError_t launch_gemm_store(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* add, const Launch& L, const Grouping& g) {
     if (ldo < w.mp || ldo % 4u) return hipErrorInvalidValue;
     return run_gemm(w, in, EpiStore{out, ldo, add}, L, g);
+}
+
+hipError_t launch_gemm_stores(const GemmStore* g, uint32_t count, const Launch& L) {
+    if (count == 0 || count > kMaxStores) return hipErrorInvalidValue;
+    auto tiles = [&](uint32_t i, uint32_t bm, uint32_t bn) { return (g[i].w.mp + bm - 1) / bm * ((g[i].in.n + bn - 1) / bn); };
+    uint32_t tall = 0, longest = 0;
+    bool f32 = false;
+    for (uint32_t i = 0; i < count; i++) {
+        if (g[i].in.n == 0 || g[i].ldo < g[i].w.mp || g[i].ldo % 4u || !shapes_fit(g[i].w, g[i].in, g[i].w.kp)) return hipErrorInvalidValue;
+        tall += tiles(i, 128, 64), longest = longest < g[i].w.kp ? g[i].w.kp : longest, f32 = f32 || g[i].in.f32;
+    }
+    if (f32) {
+        for (uint32_t i = 0; i < count; i++) {
+            const hipError_t e = launch_gemm_store(g[i].w, g[i].in, g[i].out, g[i].ldo, nullptr, L);
+            if (e != hipSuccess) return e;
+        }
+        return hipSuccess;
+    }
+    auto go = [&](auto kernel, uint32_t bm, uint32_t bn) {
+        StoresArgs s{};
+        s.count = count;
+        bool taken[kMaxStores] = {};
+        for (uint32_t k = 0; k < count; k++) {  // the longest first
+            uint32_t best = kMaxStores;
+            for (uint32_t i = 0; i < count; i++)
+                if (!taken[i] && (best == kMaxStores || g[i].w.kp > g[best].w.kp)) best = i;
+            taken[best] = true;
+            const GemmStore& p = g[best];
+            s.a[k] = GemmArgs{p.w.d, p.w.stride, p.w.kp, p.w.mp, p.in.x, p.in.ldx, p.in.n, p.w.kp, 0, Grouping()};
+            s.e[k] = EpiStore{p.out, p.ldo, nullptr};
+            s.first[k + 1] = s.first[k] + tiles(best, bm, bn);
+        }
+        return launch_kernel(L, kFamGemm, kernel, dim3(s.first[count]), dim3(256), s);
+    };
+    if (longest > 256u && tall >= 192u) return go(gemm_bf16_stores_kernel<4, 2, 3>, 128, 64);
+    return go(gemm_bf16_stores_kernel<2, 2, 4>, 64, 64);
 }
 
 hipError_t launch_gemm_gelu_split(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* bias, uint32_t split, const Launch& L) {

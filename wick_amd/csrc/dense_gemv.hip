@@ -327,8 +327,55 @@ __global__ __launch_bounds__(256) void gemv_project_kernel(ProjectArgs a) {
     }
 }
 
+// What an attention step's partials come to, gated, as floats of LDS: a thread takes four coordinates of a head and all its partials
+// (behind the active ones lies something older: loaded, not used).
+__device__ __forceinline__ void fill_merged(const WindowMerge& m, uint32_t k, float* vec) {
+    constexpr uint32_t B = 9;
+    const WindowShape& s = m.s;
+    const uint32_t stride = s.dvp + 4u, len = s.heads * s.vdim;
+    const uint32_t pos = *m.d_pos;
+    for (uint32_t e = 4u * threadIdx.x; e < k; e += 4u * kThreads) {
+        v4f out = {0.f, 0.f, 0.f, 0.f};
+        if (e < len) {
+            const uint32_t h = e / s.vdim, d = e % s.vdim;
+            const float* parts = m.part + (size_t)h * m.splits * stride;
+            const v4f z = *reinterpret_cast<const v4f*>(m.w.p + m.w.g_at + h * s.dvp + d);
+            float top = -__builtin_inff(), sum = 0.0f;
+            for (uint32_t i0 = 0; i0 < m.splits; i0 += B) {
+                v4f v[B];
+                float2 ml[B];
+#pragma unroll
+                for (uint32_t j = 0; j < B; j++) {
+                    const float* part = parts + (size_t)(i0 + j < m.splits ? i0 + j : 0u) * stride;
+                    ml[j] = *reinterpret_cast<const float2*>(part), v[j] = *reinterpret_cast<const v4f*>(part + 4 + d);
+                }
+                uint32_t tile0;
+                const uint32_t active = s.window_tiles(pos, tile0);
+                float now = top;
+#pragma unroll
+                for (uint32_t j = 0; j < B; j++) {
+                    if (i0 + j >= active || i0 + j >= m.splits) ml[j].x = -__builtin_inff();
+                    now = fmaxf(now, ml[j].x);
+                }
+                const float keep = expf(top - now);  // (the first partial is always active)
+                out *= keep, sum *= keep, top = now;
+#pragma unroll
+                for (uint32_t j = 0; j < B; j++) {
+                    if (i0 + j >= active || i0 + j >= m.splits) continue;
+                    const float w = expf(ml[j].x - now);
+                    out += v[j] * w, sum += ml[j].y * w;
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++) out[i] = out[i] / sum / (1.0f + expf(-z[i]));
+        }
+        *reinterpret_cast<v4f*>(vec + e) = out;
+    }
+}
+
 struct SegmentArgs {
     GemvSegment s[kMaxSegments];
+    WindowMerge merge;                 // of the first segment
     uint32_t first[kMaxSegments + 1];  // workgroups of segment i: first[i] .. first[i + 1] - 1
     uint32_t count;
 };
@@ -345,10 +392,14 @@ __global__ __launch_bounds__(256) void gemv_segments_kernel(SegmentArgs a) {
     for (int r = 0; r < R; r++) rows[r] = s.w.d + (size_t)(row0 + r < s.m ? row0 + r : s.m - 1u) * k;
     Ahead<R> ahead;
     ahead.load(rows, k);
-    for (uint32_t e = 4u * tid; e < k; e += 4u * kThreads) {
-        v4f v = {0.f, 0.f, 0.f, 0.f};
-        if (e < s.vec_len) v = load_to(s.vec, e, s.vec_len);
-        *reinterpret_cast<v4f*>(vec + e) = v;
+    if (i == 0 && s.merge) {
+        fill_merged(a.merge, k, vec);
+    } else {
+        for (uint32_t e = 4u * tid; e < k; e += 4u * kThreads) {
+            v4f v = {0.f, 0.f, 0.f, 0.f};
+            if (e < s.vec_len) v = load_to(s.vec, e, s.vec_len);
+            *reinterpret_cast<v4f*>(vec + e) = v;
+        }
     }
     if (s.norm_w) {
         part_rms(vec, s.vec_len, s.parts, s.eps, vec + k);
@@ -538,7 +589,11 @@ hipError_t launch_gemv_segments(const GemvSegment* segs, uint32_t count, const L
     const uint32_t R = rows <= 1024u ? 1 : 2;
     for (uint32_t i = 0; i < count; i++) {
         const GemvSegment& s = a.s[i] = segs[i];
-        if (!s.w.d || !s.vec || !s.out || s.m == 0 || s.m > s.w.mp || s.vec_len > s.w.kp || s.w.kp % 8u || s.w.kp > kGemvMaxK || s.parts == 0 || s.vec_len % s.parts ||
+        if (s.merge) {
+            if (i != 0 || !window_merge_foldable(*s.merge) || s.merge->s.heads * s.merge->s.vdim > s.w.kp) return hipErrorInvalidValue;
+            a.merge = *s.merge;
+        }
+        if (!s.w.d || !(s.vec || s.merge) || !s.out || s.m == 0 || s.m > s.w.mp || s.vec_len > s.w.kp || s.w.kp % 8u || s.w.kp > kGemvMaxK || s.parts == 0 || s.vec_len % s.parts ||
             s.parts > 512u)
             return hipErrorInvalidValue;
         a.first[i + 1] = a.first[i] + (s.m + 4u * R - 1u) / (4u * R);

@@ -22,6 +22,41 @@ struct DenseWeight {
     size_t stride = 0;         // elements between groups (experts, blocks); 0: one group
 };
 
+// ---- grouped-query attention over a window (windowed_attention.hip) ---------------------------------------------------------------
+// Position i sees j with i - window < j <= i (window 0: every j <= i); query head h uses key / value head h / (heads / kv_heads);
+// scores are capped, the weighted values gated: out = sigmoid(gate) * sum.  The cache is a ring of `slots` positions, a multiple of 64
+// that holds a window and a portion: keys [slots][kv_heads][dqp], values in tiles of 64 positions [slots / 64][kv_heads][dvp][64],
+// zeros behind dim / vdim; bfloat16, or f32.
+constexpr uint32_t kWindowTile = 64;
+struct WindowShape {
+    uint32_t heads, kv_heads, dim, vdim;
+    uint32_t dqp, dvp;           // multiples of 32
+    uint32_t rot;                // coordinates of a head that turn, in pairs (2i, 2i + 1); even
+    uint32_t window, slots, max_seq;
+    float scale, softcap;        // softcap 0: none
+    bool f32;                    // element type of the cache
+    __host__ __device__ uint32_t first_seen(uint32_t pos) const { return window && pos + 1u > window ? pos + 1u - window : 0u; }
+    // Tiles of the window of `pos`: the first one and how many.
+    __host__ __device__ uint32_t window_tiles(uint32_t pos, uint32_t& tile0) const {
+        tile0 = first_seen(pos) / kWindowTile;
+        return pos / kWindowTile - tile0 + 1u;
+    }
+};
+// Columns of a projection [n][ldp]: q [heads][dqp], k [kv_heads][dqp], v [kv_heads][dvp], g [heads][dvp]; multiples of 4.
+struct WindowProj {
+    const float* p;
+    uint32_t ldp, q_at, k_at, v_at, g_at;
+    const float* rope;           // [max_seq][rot / 2][2]: cosine, sine
+};
+// Partial results of `splits` workgroups along the window, [n][heads][splits][dvp + 4]: {max, sum, -, -, weighted values}.
+struct WindowMerge {
+    WindowShape s;
+    WindowProj w;
+    const float* part;
+    uint32_t pos0, splits;
+    const uint32_t* d_pos;       // non-null: one token at *d_pos
+};
+
 // ---- the residual stream between two sublayers (row_ops.hip, and the prologues of dense_gemv.hip) --------------------------
 // x_out = x + g_post * y / rms(y) (y null: x_out = x), then h = g_pre * x_out / rms(x_out), optionally with a causal convolution
 // over time added: h_t + sum_j conv[j] * h_(t - taps + 1 + j).  The inputs h of the last `taps` positions live in a ring of `taps`
@@ -71,6 +106,15 @@ constexpr uint32_t kGroupTileRows = 64;
 // out[t][f] = W x (+ add[f]), f32.
 hipError_t launch_gemm_store(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* add, const Launch& L,
                              const Grouping& g = Grouping());
+// Several of the plain ones in one launch (bfloat16; the f32 model's go one by one).
+struct GemmStore {
+    DenseWeight w;
+    GemmIn in;
+    float* out;
+    uint32_t ldo;
+};
+constexpr uint32_t kMaxStores = 4;
+hipError_t launch_gemm_stores(const GemmStore* g, uint32_t count, const Launch& L);
 // out[t][f] = f < split ? gelu_tanh(W x + bias) : W x + bias, f32.
 hipError_t launch_gemm_gelu_split(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* bias, uint32_t split, const Launch& L);
 // out[t][f] = relu(W x)^2 in the activation type.
@@ -117,6 +161,7 @@ struct GemvSegment {
     const float* norm_w = nullptr; // [vec_len]
     uint32_t parts = 1;
     float eps = 0.0f;
+    const WindowMerge* merge = nullptr;  // first segment: the vector is what these partials of an attention step come to (vec is not read)
 };
 constexpr uint32_t kMaxSegments = 4;
 hipError_t launch_gemv_segments(const GemvSegment* segs, uint32_t count, const Launch& L);
@@ -240,25 +285,7 @@ bool latent_prefill_shape(uint32_t dim, uint32_t rot, uint32_t vdim, uint32_t* d
 hipError_t launch_latent_prefill(const LatentShape& s, const uint16_t* q, const uint16_t* kx, uint32_t ldk, const uint16_t* vt, uint32_t ldv, uint32_t dqp,
                                  uint32_t dvp, uint32_t n, uint32_t pos0, uint16_t* out, uint32_t ldo, uint32_t kp, const Launch& L);
 
-// ---- grouped-query attention over a window (windowed_attention.hip) ---------------------------------------------------------------
-// Position i sees j with i - window < j <= i (window 0: every j <= i); query head h uses key / value head h / (heads / kv_heads);
-// scores are capped, the weighted values gated: out = sigmoid(gate) * sum.  The cache is a ring of `slots` positions, a multiple of 64
-// that holds a window and a portion: keys [slots][kv_heads][dqp], values in tiles of 64 positions [slots / 64][kv_heads][dvp][64],
-// zeros behind dim / vdim; bfloat16, or f32.
-struct WindowShape {
-    uint32_t heads, kv_heads, dim, vdim;
-    uint32_t dqp, dvp;           // multiples of 32
-    uint32_t rot;                // coordinates of a head that turn, in pairs (2i, 2i + 1); even
-    uint32_t window, slots, max_seq;
-    float scale, softcap;        // softcap 0: none
-    bool f32;                    // element type of the cache
-};
-// Columns of a projection [n][ldp]: q [heads][dqp], k [kv_heads][dqp], v [kv_heads][dvp], g [heads][dvp]; multiples of 4.
-struct WindowProj {
-    const float* p;
-    uint32_t ldp, q_at, k_at, v_at, g_at;
-    const float* rope;           // [max_seq][rot / 2][2]: cosine, sine
-};
+// Launches of windowed attention (windowed_attention.hip).
 uint32_t window_slots(uint32_t window, uint32_t portion, uint32_t max_seq);
 bool window_prefill_shape(uint32_t dim, uint32_t vdim);   // dqp / dvp of the next function have matrix-core kernels
 void window_pads(uint32_t dim, uint32_t vdim, uint32_t* dqp, uint32_t* dvp);
@@ -269,6 +296,9 @@ hipError_t launch_window_store(const WindowShape& s, const WindowProj& w, void* 
 // *d_pos whose key and value are not in the cache yet; they are appended.
 hipError_t launch_window_attention(const WindowShape& s, const WindowProj& w, void* kc, void* vc, float* scratch, uint32_t n, uint32_t pos0,
                                    const uint32_t* d_pos, void* out, uint32_t ldo, uint32_t kp, bool out_f32, const Launch& L);
+// Partials to out[t][h * vdim ..], gated.  Foldable ones (a step's) can go into the product that reads them, GemvSegment::merge.
+hipError_t launch_window_merge(const WindowMerge& m, uint32_t n, void* out, uint32_t ldo, uint32_t kp, bool out_f32, const Launch& L);
+bool window_merge_foldable(const WindowMerge& m);
 // A prompt's queries on the matrix cores (bfloat16 cache, window_prefill_shape).
 hipError_t launch_window_prefill(const WindowShape& s, const WindowProj& w, const void* kc, const void* vc, uint32_t n, uint32_t pos0, uint16_t* out,
                                  uint32_t ldo, uint32_t kp, const Launch& L);
@@ -294,6 +324,11 @@ struct SsdProj {
 constexpr uint32_t kSsdMaxState = 512;
 // One token: convolution, state and gate; out [heads * vdim] f32.
 hipError_t launch_ssd_step(const SsdShape& s, const SsdWeights& w, const SsdProj& p, float* ring, float* state, float* out, const uint32_t* d_pos, const Launch& L);
+// The same beside a step of windowed attention over the same projection, in one launch (parallel_step.hip): `merge` describes the
+// attention's partials that are left in scratch; with one split its result is in `attended` already and merge.splits is 1.
+hipError_t launch_parallel_step(const WindowShape& s, const WindowProj& w, void* kc, void* vc, float* scratch, float* attended, uint32_t attended_len,
+                                const SsdShape& ss, const SsdWeights& sw, const SsdProj& sp, float* ring, float* state, float* out, const uint32_t* d_pos,
+                                WindowMerge* merge, const Launch& L);
 // A portion, token by token in f32 (rows: [n][channels] scratch).  out [n][ldo] f32.
 hipError_t launch_ssd_scan(const SsdShape& s, const SsdWeights& w, const SsdProj& p, float* ring, float* state, float* rows, uint32_t n, uint32_t pos0,
                            float* out, uint32_t ldo, const Launch& L);

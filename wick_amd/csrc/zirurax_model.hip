@@ -307,10 +307,13 @@ int Zirurax::enqueue_step(wick_rocm_ctx* ctx, StepMode mode) {
         const GemvIn in = stage(l.norm, true);
         MODEL_LAUNCH(launch_gemv_project(l.in, l.split, in, proj, act, L));
         if (in.row.x_out) x = in.row.x_out;
-        MODEL_LAUNCH(launch_ssd_step(l.ssd, l.ssd_w, l.ssd_proj(proj), l.ring, l.state, gated, d_pos, L));
-        MODEL_LAUNCH(launch_window_attention(l.window, l.window_proj(proj), l.keys, l.values, scratch, 1, 0, d_pos, mixed, l.left_out.kp, l.left_out.kp, true, L));
+        WindowMerge merge;
+        MODEL_LAUNCH(launch_parallel_step(l.window, l.window_proj(proj), l.keys, l.values, scratch, mixed, l.left_out.kp, l.ssd, l.ssd_w, l.ssd_proj(proj), l.ring,
+                                          l.state, gated, d_pos, &merge, L));
         GemvSegment seg[3];
         seg[0] = GemvSegment{l.left_out, D, mixed, l.c.left.heads * l.c.left.vdim, y_left};
+        if (window_merge_foldable(merge)) seg[0].merge = &merge;
+        else if (merge.splits > 1) MODEL_LAUNCH(launch_window_merge(merge, 1, mixed, l.left_out.kp, l.left_out.kp, true, L));
         seg[1] = GemvSegment{l.right_out, D, gated, l.inner(), y_right, l.ssd_norm, l.c.right.parts, eps};
         if (l.c.ff) seg[2] = GemvSegment{l.down, D, act, l.down.kp, y_mlp};
         MODEL_LAUNCH(launch_gemv_segments(seg, l.c.ff ? 3 : 2, L));
@@ -385,9 +388,10 @@ int Zirurax::prompt_pass(wick_rocm_ctx* ctx, const uint32_t* tokens, uint32_t n,
         else
             MODEL_LAUNCH(launch_ssd_chunks(l.ssd, l.ssd_w, l.ssd_proj(p_proj), l.ring, l.state, p_ssd, n, pos0, p_gated, ldg, L));
         MODEL_LAUNCH(launch_part_norm(p_gated, ldg, n, l.inner(), l.c.right.parts, l.ssd_norm, eps, p_normed, ldg, ldg, f32, L));
-        MODEL_LAUNCH(launch_gemm_store(l.left_out, GemmIn{p_mixed, lda, n, f32}, p_left, dp, nullptr, L));
-        MODEL_LAUNCH(launch_gemm_store(l.right_out, GemmIn{p_normed, ldg, n, f32}, p_right, dp, nullptr, L));
-        if (l.c.ff) MODEL_LAUNCH(launch_gemm_store(l.down, GemmIn{p_act, l.down.kp, n, f32}, p_mlp, dp, nullptr, L));
+        const GemmStore outs[3] = {{l.left_out, GemmIn{p_mixed, lda, n, f32}, p_left, dp},
+                                   {l.right_out, GemmIn{p_normed, ldg, n, f32}, p_right, dp},
+                                   {l.down, GemmIn{p_act, l.down.kp, n, f32}, p_mlp, dp}};
+        MODEL_LAUNCH(launch_gemm_stores(outs, l.c.ff ? 3 : 2, L));
         pend = pending_of(l, p_left, p_right, p_mlp);
         if (layers_out) MODEL_TRY(copy_residual(ctx, pend, x, n, layers_out + (size_t)i * n * D));
     }
