@@ -109,7 +109,10 @@ struct EpiProject {
             return;
         }
 #pragma unroll
-        for (int i = 0; i < 4; i++) a[i] = gelu_tanhf(a[i]) * b[i];
+        for (int i = 0; i < 4; i++) {
+            if constexpr (sizeof(AT) == 2) a[i] = a[i] * sigmoid_hw(1.59576912160573071176f * (a[i] + 0.044715f * a[i] * a[i] * a[i])) * b[i];
+            else a[i] = gelu_tanhf(a[i]) * b[i];
+        }
         store4(act + (size_t)t * lda + (f - split / 2u), a);
     }
 };

@@ -213,30 +213,30 @@ __device__ __forceinline__ void fill_vector(const GemvIn& in, uint32_t k, float*
     }
 }
 
-// Weight pieces of N rows that a wave requests before its workgroup's prologue: the first 1024 columns.
-template <int N>
+// Weight pieces of N rows that a wave requests before its workgroup's prologue: the first 512 P columns.
+template <int N, int P = 2>
 struct Ahead {
-    uint4 w[N][2];
+    uint4 w[N][P];
     __device__ __forceinline__ void load(const uint16_t* const (&rows)[N], uint32_t k) {
         const uint32_t at = 8u * (threadIdx.x & 63u);
 #pragma unroll
-        for (int c = 0; c < 2; c++)
+        for (int c = 0; c < P; c++)
 #pragma unroll
             for (int r = 0; r < N; r++) w[r][c] = at + 512u * c < k ? *reinterpret_cast<const uint4*>(rows[r] + at + 512u * c) : uint4{0, 0, 0, 0};
     }
 };
 
-// acc[r] += this lane's share of rows[r] . vec over [0, k); AHEAD: the first 1024 columns are in `a` already.
-template <int N, bool AHEAD>
-__device__ __forceinline__ void dot_rows(const uint16_t* const (&rows)[N], const Ahead<N>* a, const float* vec, uint32_t k, float (&acc)[N]) {
+// acc[r] += this lane's share of rows[r] . vec over [0, k); the first columns are in `a` already.
+template <int N, int P>
+__device__ __forceinline__ void dot_rows(const uint16_t* const (&rows)[N], const Ahead<N, P>& a, const float* vec, uint32_t k, float (&acc)[N]) {
     uint32_t at = 8u * (threadIdx.x & 63u);
-    if constexpr (AHEAD) {
+    {
 #pragma unroll
-        for (int c = 0; c < 2; c++) {
+        for (int c = 0; c < P; c++) {
             if (at < k) {
                 const float4 v0 = *reinterpret_cast<const float4*>(vec + at), v1 = *reinterpret_cast<const float4*>(vec + at + 4);
 #pragma unroll
-                for (int r = 0; r < N; r++) acc[r] = dot8(a->w[r][c], v0, v1, acc[r]);
+                for (int r = 0; r < N; r++) acc[r] = dot8(a.w[r][c], v0, v1, acc[r]);
             }
             at += 512u;
         }
@@ -276,7 +276,7 @@ __global__ __launch_bounds__(256) void gemv_dense_kernel(DenseArgs a) {
     float acc[R];
 #pragma unroll
     for (int r = 0; r < R; r++) acc[r] = 0.0f;
-    dot_rows<R, true>(rows, &ahead, vec, a.k, acc);
+    dot_rows(rows, ahead, vec, a.k, acc);
 #pragma unroll
     for (int r = 0; r < R; r++) {
         float v = wave_sum_f32(acc[r]);
@@ -316,7 +316,7 @@ __global__ __launch_bounds__(256) void gemv_project_kernel(ProjectArgs a) {
     float acc[R];
 #pragma unroll
     for (int r = 0; r < R; r++) acc[r] = 0.0f;
-    dot_rows<R, true>(rows, &ahead, vec, a.k, acc);
+    dot_rows(rows, ahead, vec, a.k, acc);
 #pragma unroll
     for (int r = 0; r < R; r++) acc[r] = wave_sum_f32(acc[r]);
     if (lane != 0 || row0 >= a.total) return;
@@ -375,10 +375,13 @@ __device__ __forceinline__ void fill_merged(const WindowMerge& m, uint32_t k, fl
 
 struct SegmentArgs {
     GemvSegment s[kMaxSegments];
-    WindowMerge merge;                 // of the first segment
+    WindowMerge merge;                 // of segment `merged`
+    uint32_t merged;
     uint32_t first[kMaxSegments + 1];  // workgroups of segment i: first[i] .. first[i + 1] - 1
     uint32_t count;
 };
+
+constexpr int kSegmentAhead = 8;
 
 template <int R>
 __global__ __launch_bounds__(256) void gemv_segments_kernel(SegmentArgs a) {
@@ -390,9 +393,9 @@ __global__ __launch_bounds__(256) void gemv_segments_kernel(SegmentArgs a) {
     const uint16_t* rows[R];
 #pragma unroll
     for (int r = 0; r < R; r++) rows[r] = s.w.d + (size_t)(row0 + r < s.m ? row0 + r : s.m - 1u) * k;
-    Ahead<R> ahead;
+    Ahead<R, kSegmentAhead> ahead;
     ahead.load(rows, k);
-    if (i == 0 && s.merge) {
+    if (i == a.merged) {
         fill_merged(a.merge, k, vec);
     } else {
         for (uint32_t e = 4u * tid; e < k; e += 4u * kThreads) {
@@ -410,7 +413,7 @@ __global__ __launch_bounds__(256) void gemv_segments_kernel(SegmentArgs a) {
     float acc[R];
 #pragma unroll
     for (int r = 0; r < R; r++) acc[r] = 0.0f;
-    dot_rows<R, true>(rows, &ahead, vec, k, acc);
+    dot_rows(rows, ahead, vec, k, acc);
 #pragma unroll
     for (int r = 0; r < R; r++) {
         const float v = wave_sum_f32(acc[r]);
@@ -460,7 +463,7 @@ __global__ __launch_bounds__(256) void gemv_routed_up_kernel(RoutedArgs a) {
     float acc[2 * R];
 #pragma unroll
     for (int r = 0; r < 2 * R; r++) acc[r] = 0.0f;
-    dot_rows<2 * R, true>(rows, &ahead, vec, a.k, acc);
+    dot_rows(rows, ahead, vec, a.k, acc);
     if (f0 == total) {
         const float g = wave_sum_f32(acc[0]);
         if (lane == 0) a.out[total] = 1.0f / (1.0f + expf(-g));
@@ -583,15 +586,15 @@ hipError_t launch_gemv_project(const DenseWeight& w, uint32_t split, const GemvI
 hipError_t launch_gemv_segments(const GemvSegment* segs, uint32_t count, const Launch& L) {
     if (count == 0 || count > kMaxSegments) return hipErrorInvalidValue;
     SegmentArgs a{};
-    a.count = count;
+    a.count = count, a.merged = kMaxSegments;
     uint32_t lds = 0, rows = 0;
     for (uint32_t i = 0; i < count; i++) rows += segs[i].m;
     const uint32_t R = rows <= 1024u ? 1 : 2;
     for (uint32_t i = 0; i < count; i++) {
         const GemvSegment& s = a.s[i] = segs[i];
         if (s.merge) {
-            if (i != 0 || !window_merge_foldable(*s.merge) || s.merge->s.heads * s.merge->s.vdim > s.w.kp) return hipErrorInvalidValue;
-            a.merge = *s.merge;
+            if (a.merged != kMaxSegments || !window_merge_foldable(*s.merge) || s.merge->s.heads * s.merge->s.vdim > s.w.kp) return hipErrorInvalidValue;
+            a.merge = *s.merge, a.merged = i;
         }
         if (!s.w.d || !(s.vec || s.merge) || !s.out || s.m == 0 || s.m > s.w.mp || s.vec_len > s.w.kp || s.w.kp % 8u || s.w.kp > kGemvMaxK || s.parts == 0 || s.vec_len % s.parts ||
             s.parts > 512u)

@@ -104,7 +104,7 @@ struct ConvToTiles {
     __device__ void operator()(uint32_t ch, uint32_t t0, const float (&v)[kConvTokens], uint32_t count) const {
         bf8 b;
 #pragma unroll
-        for (uint32_t i = 0; i < kConvTokens; i++) b[i] = i < count ? (__bf16)siluf(v[i]) : (__bf16)0.0f;
+        for (uint32_t i = 0; i < kConvTokens; i++) b[i] = i < count ? (__bf16)(v[i] * sigmoid_hw(v[i])) : (__bf16)0.0f;
         if (ch < xs + gn) *reinterpret_cast<bf8*>(tiles + ((size_t)(t0 / kChunk) * (xs + gn) + ch) * kChunk + t0 % kChunk) = b;
         if (ch >= xs) {
 #pragma unroll
@@ -284,7 +284,7 @@ __global__ __launch_bounds__(256) void ssd_outputs_kernel(ChunkArgs a) {
 #pragma unroll
         for (int r = 0; r < 4; r++) {
             const float x = __uint_as_float((uint32_t)a.tile(c, h * s.pp + p + r)[i] << 16);
-            y[r] = (o[r] + past * q[r] + dskip * x) * siluf(z[r]);
+            y[r] = (o[r] + past * q[r] + dskip * x) * (z[r] * sigmoid_hw(z[r]));
         }
         if (s.vdim % 4u == 0) {
             if (p < s.vdim) *reinterpret_cast<v4f*>(out) = y;

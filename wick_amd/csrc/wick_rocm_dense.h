@@ -161,7 +161,7 @@ struct GemvSegment {
     const float* norm_w = nullptr; // [vec_len]
     uint32_t parts = 1;
     float eps = 0.0f;
-    const WindowMerge* merge = nullptr;  // first segment: the vector is what these partials of an attention step come to (vec is not read)
+    const WindowMerge* merge = nullptr;  // at most one segment: the vector is what these partials of an attention step come to (vec is not read)
 };
 constexpr uint32_t kMaxSegments = 4;
 hipError_t launch_gemv_segments(const GemvSegment* segs, uint32_t count, const Launch& L);

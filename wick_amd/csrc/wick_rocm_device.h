@@ -282,6 +282,9 @@ __device__ __forceinline__ float groups_sum(float v) {
 // last bit or two; the streaming softmax of this kernel differs from the reference's two-pass one at that level anyway.
 __device__ __forceinline__ float exp_nonpos_hw(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896340736f); }
 
+// Sigmoid on the hardware's exp2 and reciprocal (about two ulp), for results that leave as bfloat16.
+__device__ __forceinline__ float sigmoid_hw(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.44269504088896340736f)); }
+
 // The greedy pick's ordering (cpu_argmax, wick/src/sampler.rs:7-19) as one unsigned key: NaN counts as -inf, values order
 // by f32::total_cmp, and of equal values the larger index wins; 0 is below every real key.
 __device__ __forceinline__ unsigned long long argmax_key(float f, uint32_t index) {

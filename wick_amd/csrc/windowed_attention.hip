@@ -108,7 +108,7 @@ struct PrefillArgs {
     WindowProj w;
     const uint16_t *kc, *vc;
     uint32_t n, pos0;
-    float scale, cap, cap_inv;  // weights are exp2(cap * tanh(score * cap_inv)), without a cap exp2(score): in units of log 2
+    float scale, cap, cap_inv;  // in units of log 2: a score is scaled, then, with a cap, cap * tanh of half of score * cap_inv
     uint16_t* out;
     uint32_t ldo, kp;
 };
@@ -118,7 +118,8 @@ struct PrefillArgs {
 //   query l % 16; values transposed: O^T[d][query] += V^T[d][key] P[key][query]: the weights go from one product into the next in the
 //   registers they are in -- slot j of lane group g stands for key 4 g + j of a 16-key sub-tile (j < 4) or of the next one (j >= 4) in
 //   both operands.  The weights enter as two bfloat16 terms, so they keep 16 bits.
-template <int NS, int NV>
+// BOUNDED: the cap itself serves as the maximum of every row's scores.
+template <int NS, int NV, bool BOUNDED>
 __global__ __launch_bounds__(256) void window_prefill_kernel(PrefillArgs a) {
     constexpr uint32_t DQ = 32 * NS, DV = 16 * NV, LDK = DQ + 8, LDV = 72;
     __shared__ __align__(16) uint16_t ks[64 * LDK], vs[DV * LDV];
@@ -190,36 +191,49 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(PrefillArgs a) {
             for (int u = 0; u < 4; u++) sc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[u], qh[i], sc[u], 0, 0, 0);
         }
         const bool masked = t0 + 63u > wave_first || t0 < wave_lo_last;
-        float top = -__builtin_inff();
+        auto out_of_sight = [&](int u, int r) {
+            const uint32_t p = t0 + 16u * u + 4u * g + r;
+            return masked && (p > pq || p < lo_key);
+        };
+        float m_sub = 0.0f;
+        if constexpr (BOUNDED) {  // cap tanh(x) - cap = -2 cap / (1 + exp(2 x))
 #pragma unroll
-        for (int u = 0; u < 4; u++)
+            for (int u = 0; u < 4; u++)
 #pragma unroll
-            for (int r = 0; r < 4; r++) {
-                float v = sc[u][r] * a.scale;
-                if (a.cap > 0.0f) v = fmaf(-2.0f * a.cap, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(v * a.cap_inv)), a.cap);
-                const uint32_t p = t0 + 16u * u + 4u * g + r;
-                if (masked && (p > pq || p < lo_key)) v = -__builtin_inff();
-                sc[u][r] = v;
-                top = fmaxf(top, v);
-            }
-        top = groups_max(top);
-        const float m_new = fmaxf(m_run, top), m_sub = m_new == -__builtin_inff() ? 0.0f : m_new;
-        const float alpha = __builtin_amdgcn_exp2f(m_run - m_sub);
-        m_run = m_new;
-        float sum = 0.0f;
+                for (int r = 0; r < 4; r++) {
+                    const float v = -2.0f * a.cap * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sc[u][r] * a.cap_inv));
+                    sc[u][r] = out_of_sight(u, r) ? -__builtin_inff() : v;
+                }
+        } else {
+            float top = -__builtin_inff();
+#pragma unroll
+            for (int u = 0; u < 4; u++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    float v = sc[u][r] * a.scale;
+                    if (a.cap > 0.0f) v = fmaf(-2.0f * a.cap, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sc[u][r] * a.cap_inv)), a.cap);
+                    if (out_of_sight(u, r)) v = -__builtin_inff();
+                    sc[u][r] = v;
+                    top = fmaxf(top, v);
+                }
+            top = groups_max(top);
+            const float m_new = fmaxf(m_run, top);
+            m_sub = m_new == -__builtin_inff() ? 0.0f : m_new;
+            const float alpha = __builtin_amdgcn_exp2f(m_run - m_sub);
+            m_run = m_new, l_run *= alpha;
+#pragma unroll
+            for (int i = 0; i < NV; i++) o[i] *= alpha;
+        }
         bf8 ph[2], pl[2];
 #pragma unroll
         for (int u = 0; u < 4; u++)
 #pragma unroll
             for (int r = 0; r < 4; r++) {
                 const float p = __builtin_amdgcn_exp2f(sc[u][r] - m_sub);
-                sum += p;
+                l_run += p;
                 const __bf16 hi = (__bf16)p;
                 ph[u >> 1][4 * (u & 1) + r] = hi, pl[u >> 1][4 * (u & 1) + r] = (__bf16)(p - (float)hi);
             }
-        l_run = l_run * alpha + sum;
-#pragma unroll
-        for (int i = 0; i < NV; i++) o[i] *= alpha;
 #pragma unroll
         for (int u = 0; u < 2; u++)
 #pragma unroll
@@ -241,7 +255,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(PrefillArgs a) {
             const v4f z = *reinterpret_cast<const v4f*>(gate + d);
             v4f y;
 #pragma unroll
-            for (int r = 0; r < 4; r++) y[r] = o[i][r] * inv / (1.0f + expf(-z[r]));
+            for (int r = 0; r < 4; r++) y[r] = o[i][r] * inv * sigmoid_hw(z[r]);
             if (s.vdim % 4u == 0) {
                 const bf4 b = {(__bf16)y[0], (__bf16)y[1], (__bf16)y[2], (__bf16)y[3]};
                 if (d < s.vdim) *reinterpret_cast<bf4*>(out + d) = b;
@@ -308,17 +322,21 @@ hipError_t launch_window_prefill(const WindowShape& s, const WindowProj& w, cons
     if (n == 0) return hipSuccess;
     if (!window_shape_ok(s, w, n, pos0, true) || s.f32 || ldo < kp || kp < s.heads * s.vdim || ldo % 4u) return hipErrorInvalidValue;
     PrefillArgs a{s, w, static_cast<const uint16_t*>(kc), static_cast<const uint16_t*>(vc), n, pos0, s.scale * kLog2e, 0.0f, 0.0f, out, ldo, kp};
-    if (s.softcap > 0.0f) {  // tanh(x) = 1 - 2 / (1 + exp(2 x))
-        a.scale = s.scale, a.cap = s.softcap * kLog2e, a.cap_inv = 2.0f * kLog2e / s.softcap;
-    }
+    if (s.softcap > 0.0f) a.cap = s.softcap * kLog2e, a.cap_inv = 2.0f * kLog2e * s.scale / s.softcap;  // tanh(x) = 1 - 2 / (1 + exp(2 x))
+    const bool bounded = s.softcap > 0.0f && a.cap <= 48.0f;  // weights from exp2(-2 cap) on: far from the end of the f32 range
     const dim3 grid(s.heads, (n + 63u) / 64u);
     auto go = [&](auto ns) {
         constexpr int NS = decltype(ns)::value;
+        auto run = [&](auto nv) {
+            constexpr int NV = decltype(nv)::value;
+            return bounded ? launch_kernel(L, kFamOther, window_prefill_kernel<NS, NV, true>, grid, dim3(256), a)
+                           : launch_kernel(L, kFamOther, window_prefill_kernel<NS, NV, false>, grid, dim3(256), a);
+        };
         switch (s.dvp) {
-            case 64: return launch_kernel(L, kFamOther, window_prefill_kernel<NS, 4>, grid, dim3(256), a);
-            case 96: return launch_kernel(L, kFamOther, window_prefill_kernel<NS, 6>, grid, dim3(256), a);
-            case 128: return launch_kernel(L, kFamOther, window_prefill_kernel<NS, 8>, grid, dim3(256), a);
-            case 256: return launch_kernel(L, kFamOther, window_prefill_kernel<NS, 16>, grid, dim3(256), a);
+            case 64: return run(std::integral_constant<int, 4>{});
+            case 96: return run(std::integral_constant<int, 6>{});
+            case 128: return run(std::integral_constant<int, 8>{});
+            case 256: return run(std::integral_constant<int, 16>{});
             default: return hipErrorInvalidValue;
         }
     };

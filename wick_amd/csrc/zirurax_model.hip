@@ -310,13 +310,14 @@ int Zirurax::enqueue_step(wick_rocm_ctx* ctx, StepMode mode) {
         WindowMerge merge;
         MODEL_LAUNCH(launch_parallel_step(l.window, l.window_proj(proj), l.keys, l.values, scratch, mixed, l.left_out.kp, l.ssd, l.ssd_w, l.ssd_proj(proj), l.ring,
                                           l.state, gated, d_pos, &merge, L));
-        GemvSegment seg[3];
-        seg[0] = GemvSegment{l.left_out, D, mixed, l.c.left.heads * l.c.left.vdim, y_left};
-        if (window_merge_foldable(merge)) seg[0].merge = &merge;
+        GemvSegment left{l.left_out, D, mixed, l.c.left.heads * l.c.left.vdim, y_left};
+        if (window_merge_foldable(merge)) left.merge = &merge;
         else if (merge.splits > 1) MODEL_LAUNCH(launch_window_merge(merge, 1, mixed, l.left_out.kp, l.left_out.kp, true, L));
-        seg[1] = GemvSegment{l.right_out, D, gated, l.inner(), y_right, l.ssd_norm, l.c.right.parts, eps};
-        if (l.c.ff) seg[2] = GemvSegment{l.down, D, act, l.down.kp, y_mlp};
-        MODEL_LAUNCH(launch_gemv_segments(seg, l.c.ff ? 3 : 2, L));
+        std::vector<GemvSegment> outs;  // the longest first
+        if (l.c.ff) outs.push_back(GemvSegment{l.down, D, act, l.down.kp, y_mlp});
+        outs.push_back(left);
+        outs.push_back(GemvSegment{l.right_out, D, gated, l.inner(), y_right, l.ssd_norm, l.c.right.parts, eps});
+        MODEL_LAUNCH(launch_gemv_segments(outs.data(), (uint32_t)outs.size(), L));
         pend = pending_of(l, y_left, y_right, y_mlp);
     }
     return finish_step(ctx, mode, stage(final_norm.w, false));
