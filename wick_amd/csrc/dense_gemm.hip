@@ -3,10 +3,11 @@
 //
 // Two bodies share the epilogues, because the 16 x 16 result of v_mfma_f32_16x16x32_bf16 and of v_mfma_f32_16x16x4_f32 sits in the
 // same registers (lane l: column l % 16, rows 4 (l / 16) + r):
-//   gemm_bf16_kernel  activations in bfloat16; 2 x 2 waves of (16 MT) x (16 NT) outputs, K in steps of 64 through two LDS buffers
+//   gemm_bf16_kernel  activations in bfloat16; WM x WN waves of (16 MT) x (16 NT) outputs, K in steps of 64 through two LDS buffers
 //                     (the global loads of the next PD steps are in flight during the products of this one: a tile of a small
-//                     product is alone on its CU, and a step's products are much shorter than a trip to memory); the 16-byte chunks of an LDS
-//                     row are permuted by row % 8, so that the 16 rows a fragment read touches spread over the banks;
+//                     product is alone on its CU, and a step's products are much shorter than a trip to memory; the tiles of a large one
+//                     are shared by sixteen waves, which hide the trips themselves and read every operand half as often); the 16-byte
+//                     chunks of an LDS row are permuted by row % 8, so that the 16 rows a fragment read touches spread over the banks;
 //   gemm_f32_kernel   activations in f32, weights widened exactly: every product and sum in f32.
 // Weights are the M side, so a lane ends with four consecutive features of one token: one vector store.  With TRANS the sides are
 // swapped and a lane holds four consecutive tokens of one feature (a transposed result).
@@ -221,27 +222,27 @@ __device__ __forceinline__ void run_epilogue(const GemmArgs& a, const TileAt& o,
 }
 
 // Tile `bid` of `count`.
-template <int MT, int NT, int PD, class Epi>
+template <int MT, int NT, int PD, int WM, int WN, class Epi>
 __device__ __forceinline__ void gemm_bf16_tile(const GemmArgs& a, const Epi& epi, uint32_t bid, uint32_t count) {
-    constexpr uint32_t BM = 32 * MT, BN = 32 * NT, BK = 64;
-    constexpr int LA = BM * 8 / 256, LB = BN * 8 / 256;  // 16-byte chunks per thread and step
+    constexpr uint32_t BM = 16 * MT * WM, BN = 16 * NT * WN, BK = 64, THREADS = 64 * WM * WN;
+    constexpr int LA = BM * 8 / THREADS, LB = BN * 8 / THREADS;  // 16-byte chunks per thread and step
     __shared__ __align__(16) uint16_t sa[2][BM * BK], sb[2][BN * BK];
     TileAt o;
     if (!tile_at(a, BM, BN, bid, count, o)) return;
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, g = lane >> 4;
-    const uint32_t wm = (wave & 1u) * (16 * MT), wn = (wave >> 1) * (16 * NT);
+    const uint32_t wm = (wave % WM) * (16 * MT), wn = (wave / WM) * (16 * NT);
     const uint16_t* x = static_cast<const uint16_t*>(a.x) + (size_t)o.z * a.x_stride_z;
     const uint16_t *pa[LA], *pb[LB];
     uint32_t da[LA], db[LB];
 #pragma unroll
     for (int i = 0; i < LA; i++) {
-        const uint32_t c = tid + 256 * i, row = c >> 3, ch = c & 7u, m = o.m0 + row < a.mp ? o.m0 + row : a.mp - 1u;
+        const uint32_t c = tid + THREADS * i, row = c >> 3, ch = c & 7u, m = o.m0 + row < a.mp ? o.m0 + row : a.mp - 1u;
         pa[i] = o.w + (size_t)m * a.ldw + ch * 8;
         da[i] = row * BK + ((ch ^ (row & 7u)) << 3);
     }
 #pragma unroll
     for (int i = 0; i < LB; i++) {
-        const uint32_t c = tid + 256 * i, row = c >> 3, ch = c & 7u;
+        const uint32_t c = tid + THREADS * i, row = c >> 3, ch = c & 7u;
         pb[i] = x + (size_t)source_row(a, o, row) * a.ldx + ch * 8;
         db[i] = row * BK + ((ch ^ (row & 7u)) << 3);
     }
@@ -303,9 +304,9 @@ __device__ __forceinline__ void gemm_bf16_tile(const GemmArgs& a, const Epi& epi
     run_epilogue<MT, NT>(a, o, epi, acc, wm, wn, l16, g);
 }
 
-template <int MT, int NT, int PD, class Epi>
-__global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
-    gemm_bf16_tile<MT, NT, PD>(a, epi, blockIdx.x, gridDim.x);
+template <int MT, int NT, int PD, int WM, int WN, class Epi>
+__global__ __launch_bounds__(64 * WM * WN) void gemm_bf16_kernel(GemmArgs a, Epi epi) {
+    gemm_bf16_tile<MT, NT, PD, WM, WN>(a, epi, blockIdx.x, gridDim.x);
 }
 
 struct StoresArgs {
@@ -313,11 +314,11 @@ struct StoresArgs {
     EpiStore e[kMaxStores];
     uint32_t first[kMaxStores + 1], count;  // tiles of product i: first[i] .. first[i + 1] - 1
 };
-template <int MT, int NT, int PD>
-__global__ __launch_bounds__(256) void gemm_bf16_stores_kernel(StoresArgs s) {
+template <int MT, int NT, int PD, int WM, int WN>
+__global__ __launch_bounds__(64 * WM * WN) void gemm_bf16_stores_kernel(StoresArgs s) {
     uint32_t i = 0;
     while (i + 1 < s.count && blockIdx.x >= s.first[i + 1]) i++;
-    gemm_bf16_tile<MT, NT, PD>(s.a[i], s.e[i], blockIdx.x - s.first[i], s.first[i + 1] - s.first[i]);
+    gemm_bf16_tile<MT, NT, PD, WM, WN>(s.a[i], s.e[i], blockIdx.x - s.first[i], s.first[i + 1] - s.first[i]);
 }
 
 template <class Epi>
@@ -383,12 +384,13 @@ hipError_t run_gemm(const DenseWeight& w, const GemmIn& in, const Epi& epi, cons
         return dim3(mt * nt, 1, z);
     };
     if (in.f32) return launch_kernel(L, kFamGemm, gemm_f32_kernel<Epi>, grid(64, 64), dim3(256), a, epi);
-    if (g.tiles) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, 3, Epi>, grid(128, kGroupTileRows), dim3(256), a, epi);
+    if (g.tiles) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, 3, 2, 2, Epi>, grid(128, kGroupTileRows), dim3(256), a, epi);
     // the widest tile that leaves no CU without one (a short K is mostly epilogue: small tiles, more of them)
-    const dim3 big = grid(128, 128), tall = grid(128, 64);
-    if (w.kp > 256u && big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, 2, Epi>, big, dim3(256), a, epi);
-    if (w.kp > 256u && tall.x * tall.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, 3, Epi>, tall, dim3(256), a, epi);
-    return launch_kernel(L, kFamGemm, gemm_bf16_kernel<2, 2, 4, Epi>, grid(64, 64), dim3(256), a, epi);
+    const dim3 huge = grid(256, 256), big = grid(128, 128), tall = grid(128, 64);
+    if (w.kp > 256u && huge.x * huge.z >= 320u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, 1, 4, 4, Epi>, huge, dim3(1024), a, epi);
+    if (w.kp > 256u && big.x * big.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 4, 2, 2, 2, Epi>, big, dim3(256), a, epi);
+    if (w.kp > 256u && tall.x * tall.z >= 192u) return launch_kernel(L, kFamGemm, gemm_bf16_kernel<4, 2, 3, 2, 2, Epi>, tall, dim3(256), a, epi);
+    return launch_kernel(L, kFamGemm, gemm_bf16_kernel<2, 2, 4, 2, 2, Epi>, grid(64, 64), dim3(256), a, epi);
 }
 
 }  // namespace
@@ -414,7 +416,7 @@ hipError_t launch_gemm_stores(const GemmStore* g, uint32_t count, const Launch& 
         }
         return hipSuccess;
     }
-    auto go = [&](auto kernel, uint32_t bm, uint32_t bn) {
+    auto go = [&](auto kernel, uint32_t bm, uint32_t bn, uint32_t threads) {
         StoresArgs s{};
         s.count = count;
         bool taken[kMaxStores] = {};
@@ -428,10 +430,10 @@ hipError_t launch_gemm_stores(const GemmStore* g, uint32_t count, const Launch& 
             s.e[k] = EpiStore{p.out, p.ldo, nullptr};
             s.first[k + 1] = s.first[k] + tiles(best, bm, bn);
         }
-        return launch_kernel(L, kFamGemm, kernel, dim3(s.first[count]), dim3(256), s);
+        return launch_kernel(L, kFamGemm, kernel, dim3(s.first[count]), dim3(threads), s);
     };
-    if (longest > 256u && tall >= 192u) return go(gemm_bf16_stores_kernel<4, 2, 3>, 128, 64);
-    return go(gemm_bf16_stores_kernel<2, 2, 4>, 64, 64);
+    if (longest > 256u && tall >= 192u) return go(gemm_bf16_stores_kernel<2, 2, 1, 4, 2>, 128, 64, 512);
+    return go(gemm_bf16_stores_kernel<2, 2, 4, 2, 2>, 64, 64, 256);
 }
 
 hipError_t launch_gemm_gelu_split(const DenseWeight& w, const GemmIn& in, float* out, uint32_t ldo, const float* bias, uint32_t split, const Launch& L) {
