@@ -213,6 +213,12 @@ __device__ __forceinline__ void fill_vector(const GemvIn& in, uint32_t k, float*
     }
 }
 
+__device__ __forceinline__ uint4 stream_load(const uint16_t* p) {
+    typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+    const u4 v = __builtin_nontemporal_load(reinterpret_cast<const u4*>(p));
+    return uint4{v[0], v[1], v[2], v[3]};
+}
+
 // Weight pieces of N rows that a wave requests before its workgroup's prologue: the first 512 P columns.
 template <int N, int P = 2>
 struct Ahead {
@@ -222,7 +228,7 @@ struct Ahead {
 #pragma unroll
         for (int c = 0; c < P; c++)
 #pragma unroll
-            for (int r = 0; r < N; r++) w[r][c] = at + 512u * c < k ? *reinterpret_cast<const uint4*>(rows[r] + at + 512u * c) : uint4{0, 0, 0, 0};
+            for (int r = 0; r < N; r++) w[r][c] = at + 512u * c < k ? stream_load(rows[r] + at + 512u * c) : uint4{0, 0, 0, 0};
     }
 };
 
@@ -245,7 +251,7 @@ __device__ __forceinline__ void dot_rows(const uint16_t* const (&rows)[N], const
     for (; at < k; at += 512u) {
         uint4 w[N];
 #pragma unroll
-        for (int r = 0; r < N; r++) w[r] = *reinterpret_cast<const uint4*>(rows[r] + at);
+        for (int r = 0; r < N; r++) w[r] = stream_load(rows[r] + at);
         const float4 v0 = *reinterpret_cast<const float4*>(vec + at), v1 = *reinterpret_cast<const float4*>(vec + at + 4);
 #pragma unroll
         for (int r = 0; r < N; r++) acc[r] = dot8(w[r], v0, v1, acc[r]);

@@ -16,6 +16,7 @@ using namespace folder_model;
 
 constexpr uint32_t kChunkBf16 = 2048, kChunkExact = 512;  // tokens per prompt pass: bfloat16 / f32 or heads without matrix-core attention
 constexpr uint32_t kShortMax = 16;                        // portions this short run token by token through attention and state
+constexpr uint32_t kForkMin = 256;                        // longer portions run attention and state side by side
 
 struct AttentionConfig {
     uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, window = 0, rot = 0;
@@ -68,6 +69,16 @@ struct Zirurax final : FolderModel {
     void *p_act = nullptr, *p_mixed = nullptr, *p_normed = nullptr;
     SsdScratch p_ssd{};
 
+    // a prompt pass's state-space side runs beside its attention
+    hipStream_t side = nullptr;
+    hipEvent_t projected = nullptr, scanned = nullptr;
+
+    void release(wick_rocm_ctx* ctx) override {
+        if (side) (void)hipStreamSynchronize(side), (void)hipStreamDestroy(side);
+        if (projected) (void)hipEventDestroy(projected);
+        if (scanned) (void)hipEventDestroy(scanned);
+        FolderModel::release(ctx);
+    }
     bool exact(const Layer& l) const { return f32 || !window_prefill_shape(l.c.left.dim, l.c.left.vdim); }
     int load(wick_rocm_ctx* ctx, const wick_safetensors* folder, uint32_t context_size);
     int load_layer(wick_rocm_ctx* ctx, const wick_safetensors* folder, uint32_t i);
@@ -359,6 +370,9 @@ int Zirurax::alloc_rows(wick_rocm_ctx* ctx) {
         MODEL_TRY(alloc_t(ctx, sums_n, &p_ssd.sums));
         MODEL_TRY(alloc_t(ctx, 2 * sums_n, &p_ssd.starts));
     }
+    MODEL_LAUNCH(hipStreamCreateWithFlags(&side, hipStreamNonBlocking));
+    MODEL_LAUNCH(hipEventCreateWithFlags(&projected, hipEventDisableTiming));
+    MODEL_LAUNCH(hipEventCreateWithFlags(&scanned, hipEventDisableTiming));
     cap = pass;
     return WICK_ROCM_OK;
 }
@@ -379,16 +393,25 @@ int Zirurax::prompt_pass(wick_rocm_ctx* ctx, const uint32_t* tokens, uint32_t n,
         MODEL_LAUNCH(launch_gemm_project(l.in, GemmIn{p_h, dp, n, f32}, l.split, p_proj, l.split, p_act, l.down.kp, L));
         const WindowProj w = l.window_proj(p_proj);
         const uint32_t lda = l.left_out.kp, ldg = l.right_out.kp;
+        const bool fork = n > kForkMin && !(L.timer && L.timer->enabled);
+        Launch S = L;
+        if (fork) {
+            S.stream = side;
+            MODEL_LAUNCH(hipEventRecord(projected, L.stream));
+            MODEL_LAUNCH(hipStreamWaitEvent(side, projected, 0));
+        }
+        if (f32 || n <= kShortMax)
+            MODEL_LAUNCH(launch_ssd_scan(l.ssd, l.ssd_w, l.ssd_proj(p_proj), l.ring, l.state, p_conv, n, pos0, p_gated, ldg, S));
+        else
+            MODEL_LAUNCH(launch_ssd_chunks(l.ssd, l.ssd_w, l.ssd_proj(p_proj), l.ring, l.state, p_ssd, n, pos0, p_gated, ldg, S));
+        MODEL_LAUNCH(launch_part_norm(p_gated, ldg, n, l.inner(), l.c.right.parts, l.ssd_norm, eps, p_normed, ldg, ldg, f32, S));
+        if (fork) MODEL_LAUNCH(hipEventRecord(scanned, side));
         MODEL_LAUNCH(launch_window_store(l.window, w, l.keys, l.values, n, pos0, L));
         if (exact(l) || n <= kShortMax)
             MODEL_LAUNCH(launch_window_attention(l.window, w, l.keys, l.values, p_scratch, n, pos0, nullptr, p_mixed, lda, lda, f32, L));
         else
             MODEL_LAUNCH(launch_window_prefill(l.window, w, l.keys, l.values, n, pos0, static_cast<uint16_t*>(p_mixed), lda, lda, L));
-        if (f32 || n <= kShortMax)
-            MODEL_LAUNCH(launch_ssd_scan(l.ssd, l.ssd_w, l.ssd_proj(p_proj), l.ring, l.state, p_conv, n, pos0, p_gated, ldg, L));
-        else
-            MODEL_LAUNCH(launch_ssd_chunks(l.ssd, l.ssd_w, l.ssd_proj(p_proj), l.ring, l.state, p_ssd, n, pos0, p_gated, ldg, L));
-        MODEL_LAUNCH(launch_part_norm(p_gated, ldg, n, l.inner(), l.c.right.parts, l.ssd_norm, eps, p_normed, ldg, ldg, f32, L));
+        if (fork) MODEL_LAUNCH(hipStreamWaitEvent(L.stream, scanned, 0));
         const GemmStore outs[3] = {{l.left_out, GemmIn{p_mixed, lda, n, f32}, p_left, dp},
                                    {l.right_out, GemmIn{p_normed, ldg, n, f32}, p_right, dp},
                                    {l.down, GemmIn{p_act, l.down.kp, n, f32}, p_mlp, dp}};
