@@ -251,6 +251,40 @@ def test_the_ring_of_keys_and_values_goes_round(ctx, tmp_path, dtype):
         p.check(got[places], want[places])
 
 
+@BOTH
+def test_one_key_thousands_of_positions_back(ctx, tmp_path, dtype):
+    """Without a window: more tiles than a step has workgroups along the sequence, a key that stands out in the first and in the last of
+    them, and between; in a step and in prompt passes."""
+    cfg = S.config([S.layer(S.attention(heads=2, kv_heads=1, dim=16, vdim=16, window=None, turn=S.rot(2, 1e7, None), scale=3.0, softcap=60.0),
+                            S.ssd(heads=1, groups=1, state=4, vdim=4), ff=None)], width=64, vocab=64, scale=0.3)
+    t = S.tensors(cfg, 17)
+    t["l0.mix.right.out"] = t["l0.mix.right.out"] * 0
+    x, eps = t["embed"].astype(np.float64) * 0.3, cfg["norm"]["eps"]
+    h = O.rms(x, eps) * t["l0.norm1"]
+    q, k = (h @ t["l0.mix.left.q"].T).reshape(64, 2, 16), h @ t["l0.mix.left.k"].T
+    score = 60.0 * np.tanh(3.0 * np.einsum("qhd,kd->qhk", q, k) / 60.0)
+    gap = (score.max(-1) - np.median(score, -1)).min(-1)  # a query with a key far above most others, for both heads
+    query = int(np.argmax(gap))
+    key, filler = int(np.argmax(score[query].min(0))), int(np.argmin(score[query].max(0)))
+    n = 4200
+    with Pair(ctx, tmp_path, cfg, dtype, seed=17, context=n + 4, t=t) as p:
+        plain = np.full(n, filler)
+        plain[-1] = query
+        ref = last(p, plain)
+        for at in (0, 63, 64, 2050, 4095, 4096, 4160):
+            toks = plain.copy()
+            toks[at] = key
+            want = last(p, toks)
+            p.tol = TOL_F32 if dtype == F32 else 0.03  # (about ten roundings of a bfloat16 activation)
+            assert error(want, ref) > max(0.15, 5 * p.tol)
+            p.gpu.forward(toks[:-1], 0, [])
+            p.check(p.gpu.forward(toks[-1:], n - 1), want)
+            if at in (64, 4096):
+                p.check(p.gpu.forward(toks, 0, [n - 1]), want)
+                p.gpu.forward(toks[:-9], 0, [])
+                p.check(p.gpu.forward(toks[-9:], n - 9, [8]), want)
+
+
 def test_many_wanted_places(ctx, tmp_path):
     """More wanted rows than one product with the head takes, in a step each and in one pass."""
     with Pair(ctx, tmp_path, S.mixed(), NATIVE, seed=10) as p:
